@@ -19,7 +19,7 @@ from typing import Dict, List, Optional, Sequence
 import numpy as np
 import torch
 
-from ..models.configs import ModelConfig
+from ..models.configs import (ChannelDeltaSpec, LayeredConfig, ModelConfig)
 
 BLOCK_SIZE = 16  # tokens per KV block (reference default, types.go:92)
 
@@ -81,6 +81,15 @@ class KVPool:
     def layer(self, li: int):
         return self.tensor[li, 0], self.tensor[li, 1]
 
+    def model_view(self) -> torch.Tensor:
+        """What the model's forward takes."""
+        return self.tensor
+
+    @property
+    def transfer_view(self) -> torch.Tensor:
+        """The blocks the transfer engine moves between ranks."""
+        return self.tensor
+
     @property
     def block_bytes(self) -> int:
         """Bytes of one block across all layers and K+V."""
@@ -97,13 +106,82 @@ class KVPool:
         return max(16, budget_bytes // per_block)
 
 
+class LayeredPool:
+    """Cache of a layer-listed design. A latent-attention layer that owns its
+    latents has pages [num_blocks, block_size, kv_rank + rot_dim] (layers
+    that attend to another layer's latents have none); a recurrent layer has
+    one slot per live sequence: convolution inputs [slots, taps - 1,
+    channels] and the matrix state [slots, heads, dim, vdim] in 32-bit.
+
+    Slots are never cleared: the kernels start a sequence without earlier
+    tokens from zero."""
+
+    def __init__(self, config: LayeredConfig, num_blocks: int,
+                 state_slots: int, device: torch.device, dtype: torch.dtype,
+                 block_size: int = BLOCK_SIZE):
+        self.cfg = config
+        self.num_blocks = num_blocks
+        self.block_size = block_size
+        self.device = device
+        self.dtype = self.cache_dtype = dtype
+        self.state_slots = state_slots if config.has_recurrent_state else 0
+        self.ipc_backed = False
+        self.layers: List[object] = []
+        for layer in config.layers:
+            m = layer.mixer
+            if isinstance(m, ChannelDeltaSpec):
+                state, conv = m.state_shapes
+                self.layers.append((
+                    torch.zeros((state_slots,) + conv, dtype=dtype,
+                                device=device),
+                    torch.zeros((state_slots,) + state, dtype=torch.float32,
+                                device=device)))
+            elif m.cache_width:
+                self.layers.append(torch.zeros(
+                    (num_blocks, block_size, m.cache_width), dtype=dtype,
+                    device=device))
+            else:
+                self.layers.append(None)
+
+    def model_view(self) -> "LayeredPool":
+        return self
+
+    @property
+    def transfer_view(self) -> torch.Tensor:
+        """No hand-off between ranks: an empty pool of the usual rank."""
+        return torch.empty((0, 2, self.num_blocks, 1, self.block_size, 0),
+                           dtype=self.dtype, device=self.device)
+
+    @property
+    def block_bytes(self) -> int:
+        return self.block_size * self.cfg.kv_bytes_per_token(
+            self.dtype.itemsize)
+
+    @staticmethod
+    def plan(config: LayeredConfig, budget_bytes: int, max_slots: int,
+             block_size: int = BLOCK_SIZE, dtype_bytes: int = 2):
+        """Split a budget -> (blocks, state slots): up to half of it for
+        state, the rest for pages."""
+        per_seq = config.state_bytes_per_sequence(dtype_bytes)
+        slots = max_slots
+        if per_seq:
+            slots = max(1, min(max_slots, budget_bytes // 2 // per_seq))
+        per_block = max(1, block_size * config.kv_bytes_per_token(
+            dtype_bytes))
+        return max(16, (budget_bytes - slots * per_seq) // per_block), slots
+
+
 class BlockManager:
     """Refcounted free-list allocator + per-sequence block tables with
-    content-addressed full-block prefix caching."""
+    content-addressed full-block prefix caching. With `state_slots`, every
+    sequence that holds blocks also holds one recurrent-state slot."""
 
     def __init__(self, num_blocks: int, block_size: int = BLOCK_SIZE,
-                 prefix_caching: bool = True):
+                 prefix_caching: bool = True, state_slots: int = 0):
         self.num_blocks = num_blocks
+        self.state_slots = state_slots
+        self._free_slots: List[int] = list(range(state_slots - 1, -1, -1))
+        self.slot_of: Dict[str, int] = {}
         self.block_size = block_size
         self.prefix_caching = prefix_caching
         # all blocks start free and content-less; LRU order: oldest first
@@ -205,6 +283,9 @@ class BlockManager:
         prefix is most of the pool (found by the engine-lifecycle
         property fuzz)."""
         need = (n_tokens + self.block_size - 1) // self.block_size
+        if self.state_slots and not self._free_slots and \
+                seq_id not in self.slot_of:
+            return False
         if seq_id is not None:
             need -= len(self.tables.get(seq_id, ()))
         return need <= len(self._free_lru)
@@ -213,11 +294,20 @@ class BlockManager:
         """Ensure the sequence has capacity for n_tokens total."""
         table = self.tables.setdefault(seq_id, [])
         need = (n_tokens + self.block_size - 1) // self.block_size
-        if need - len(table) > len(self._free_lru):
+        if need - len(table) > len(self._free_lru) or \
+                not self._take_slot(seq_id):
             return False
         while len(table) < need:
             table.append(self._pop_free())
         self.seq_lens.setdefault(seq_id, 0)
+        return True
+
+    def _take_slot(self, seq_id: str) -> bool:
+        if not self.state_slots or seq_id in self.slot_of:
+            return True
+        if not self._free_slots:
+            return False
+        self.slot_of[seq_id] = self._free_slots.pop()
         return True
 
     def append_token_slot(self, seq_id: str) -> Optional[int]:
@@ -242,6 +332,9 @@ class BlockManager:
         for blk in self.tables.pop(seq_id, []):
             self._release(blk)
         self.seq_lens.pop(seq_id, None)
+        slot = self.slot_of.pop(seq_id, None)
+        if slot is not None:
+            self._free_slots.append(slot)
 
     def adopt(self, seq_id: str, blocks: List[int], seq_len: int) -> None:
         """Adopt externally-filled blocks (xGMI transfer receive path)."""

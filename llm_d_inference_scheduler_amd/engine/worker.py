@@ -16,16 +16,19 @@ so step N+1 launches before step N's token values have landed.
 """
 import time
 from dataclasses import dataclass, field
-from typing import Dict, List, Optional
+from typing import Callable, Dict, List, Optional
 
 import numpy as np
 import torch
 
 from ..datalayer.endpoint import Metrics, Role
-from ..models.configs import ModelConfig
-from ..models.llama import ForwardBatch, LlamaRunner
+from ..models.configs import LayeredConfig
+from ..models.layered import SHORT, LayeredBatch, Portion
+from ..models.llama import ForwardBatch
+from ..models.registry import AnyConfig, build_runner
 from ..utils.logging import get_logger
-from .kvcache import BLOCK_SIZE, BlockManager, KVPool, block_hashes
+from .kvcache import (BLOCK_SIZE, BlockManager, KVPool, LayeredPool,
+                      block_hashes)
 
 log = get_logger("engine.worker")
 
@@ -70,6 +73,14 @@ class EngineRequest:
 
 
 @dataclass
+class TokenSpan:
+    """Given tokens of one request for one step (forward_spans)."""
+    request_id: str
+    tokens: List[int]
+    want: List[int] = field(default_factory=list)   # places needing logits
+
+
+@dataclass
 class RequestOutput:
     request_id: str
     new_tokens: List[int]
@@ -104,6 +115,7 @@ class DecodeState:
         self.seq_lens = None
         self.last_tok = None
         self.temps = None
+        self.state_slots = None     # recurrent-state slot of every row
         self.free_rows: List[int] = []
         self.row_of: Dict[str, int] = {}
         self._active_ids: List[str] = []
@@ -117,12 +129,15 @@ class DecodeState:
         sl = torch.zeros(new_cap, dtype=torch.int32, device=self.device)
         lt = torch.zeros(new_cap, dtype=torch.int64, device=self.device)
         tp = torch.zeros(new_cap, dtype=torch.float32, device=self.device)
+        ss = torch.zeros(new_cap, dtype=torch.int32, device=self.device)
         if old:
             bt[:old] = self.bt
             sl[:old] = self.seq_lens
             lt[:old] = self.last_tok
             tp[:old] = self.temps
+            ss[:old] = self.state_slots
         self.bt, self.seq_lens, self.last_tok, self.temps = bt, sl, lt, tp
+        self.state_slots = ss
         self.free_rows.extend(range(new_cap - 1, old - 1, -1))
         self.capacity = new_cap
 
@@ -132,7 +147,7 @@ class DecodeState:
         return self.free_rows.pop()
 
     def join(self, req: EngineRequest, table: List[int], seq_len: int,
-             last_token: int) -> None:
+             last_token: int, state_slot: int = 0) -> None:
         row = self.take_row()
         self.row_of[req.request_id] = row
         # any membership mutation invalidates the cached row-index tensor:
@@ -147,6 +162,7 @@ class DecodeState:
         self.seq_lens[row] = seq_len
         self.last_tok[row] = last_token
         self.temps[row] = req.temperature
+        self.state_slots[row] = state_slot
 
     def leave(self, request_id: str) -> None:
         row = self.row_of.pop(request_id, None)
@@ -165,7 +181,7 @@ class DecodeState:
 
 
 class EngineWorker:
-    def __init__(self, config: ModelConfig, device,
+    def __init__(self, config: AnyConfig, device,
                  role: Role = Role.DECODE,
                  kv_blocks: Optional[int] = None,
                  kv_budget_bytes: int = 8 << 30,
@@ -180,6 +196,7 @@ class EngineWorker:
                  prefill_max_delay_ms: float = 60.0,
                  ipc_pool: bool = False,
                  overlap_streams: Optional[bool] = None,
+                 state_slots: Optional[int] = None,
                  seed: int = 0):
         self.cfg = config
         self.device = torch.device(device)
@@ -197,16 +214,36 @@ class EngineWorker:
         if cache_dtype == torch.float8_e4m3fn and \
                 self.device.type != "cuda":
             cache_dtype = dtype     # fp8 path needs the gfx950 kernels
-        if kv_blocks is None:
-            kv_blocks = KVPool.blocks_for_budget(
-                config, kv_budget_bytes,
-                dtype_bytes=cache_dtype.itemsize)
-        self.pool = KVPool(config, kv_blocks, self.device, dtype,
-                           cache_dtype=cache_dtype,
-                           ipc_alloc=ipc_pool and self._is_cuda_dev())
-        self.mgr = BlockManager(kv_blocks, self.pool.block_size,
-                                prefix_caching=prefix_caching)
-        self.model = LlamaRunner(config, self.device, dtype, seed=seed)
+        if isinstance(config, LayeredConfig):
+            if cache_dtype != dtype:
+                raise ValueError("layer-listed designs keep their cache in "
+                                 "the compute dtype (kv_cache_dtype=auto)")
+            blocks, slots = LayeredPool.plan(config, kv_budget_bytes,
+                                             max_decode_batch,
+                                             dtype_bytes=dtype.itemsize)
+            self.pool = LayeredPool(
+                config, kv_blocks or blocks,
+                state_slots if state_slots is not None else slots,
+                self.device, dtype)
+            # a recurrent state exists only at its sequence's end: a prompt
+            # cannot start from another prompt's cached blocks
+            prefix_caching = prefix_caching and \
+                not config.has_recurrent_state
+        else:
+            if kv_blocks is None:
+                kv_blocks = KVPool.blocks_for_budget(
+                    config, kv_budget_bytes,
+                    dtype_bytes=cache_dtype.itemsize)
+            self.pool = KVPool(config, kv_blocks, self.device, dtype,
+                               cache_dtype=cache_dtype,
+                               ipc_alloc=ipc_pool and self._is_cuda_dev())
+        self.mgr = BlockManager(self.pool.num_blocks, self.pool.block_size,
+                                prefix_caching=prefix_caching,
+                                state_slots=getattr(self.pool, "state_slots",
+                                                    0))
+        self.model = build_runner(config, self.device, dtype, seed=seed,
+                                  max_model_len=max_model_len)
+        self._mixed = self.model.mixed_batches
         self.waiting: List[EngineRequest] = []
         self.running: List[EngineRequest] = []
         self._by_id: Dict[str, EngineRequest] = {}
@@ -252,6 +289,11 @@ class EngineWorker:
             # an empty prompt would be silently dropped in _prefill_pass
             # (remaining <= 0) and the client would hang until timeout
             self._reject(req, "empty_prompt: prompt tokenized to 0 tokens")
+            return
+        if self._mixed and (req.prefill_only
+                            or req.prefix_embeds is not None):
+            self._reject(req, "unsupported: this design has neither a "
+                              "hand-off between ranks nor a vision tower")
             return
         if len(req.prompt_tokens) >= self.max_model_len:
             # reject, never truncate: a silently-truncated prompt produces
@@ -353,7 +395,9 @@ class EngineWorker:
             outputs.extend(self._carry)
             self._carry = []
         do_prefill = bool(self.waiting) and self._should_prefill()
-        if self._cuda and self._overlap and do_prefill and self.running:
+        if self._mixed:
+            outputs.extend(self._mixed_pass(do_prefill))
+        elif self._cuda and self._overlap and do_prefill and self.running:
             # Overlap the two passes: decode (HBM-bound paged attention +
             # skinny GEMMs) launches first on the default stream; prefill
             # (MFMA-bound flash attention + fat GEMMs) runs concurrently
@@ -403,7 +447,9 @@ class EngineWorker:
     # ---- prefill ----
     def _admit_prompt(self, req: EngineRequest) -> None:
         """First touch: match + reuse cached prefix blocks (engine APC)."""
-        if req.block_hashes is None:
+        if not self.mgr.prefix_caching:
+            req.block_hashes = np.zeros(0, dtype=np.uint64)
+        elif req.block_hashes is None:
             req.block_hashes = block_hashes(req.prompt_tokens,
                                             self.pool.block_size)
         matched = self.mgr.allocate_prompt(req.request_id, req.block_hashes,
@@ -413,8 +459,8 @@ class EngineWorker:
         req.registered_blocks = matched // self.pool.block_size
         self.mgr.set_seq_len(req.request_id, matched)
 
-    def _prefill_pass(self) -> List[RequestOutput]:
-        budget = self.prefill_chunk_tokens
+    def _select_prefill(self, budget: int) -> List[tuple]:
+        """Admit and allocate this step's portions -> [(request, tokens)]."""
         selected: List[tuple] = []
         # priority-ordered admission (stable within a priority class):
         # a preempted victim must not re-grab blocks freed FOR a
@@ -441,6 +487,33 @@ class EngineWorker:
                 break
             selected.append((req, chunk))
             budget -= chunk
+        return selected
+
+    def _advance_prefill(self, req: EngineRequest, chunk: int) -> bool:
+        """Account for a portion that is about to run; True on its last."""
+        start, end = req.computed, req.computed + chunk
+        self.mgr.set_seq_len(req.request_id, end)
+        req.computed = end
+        self.total_prefilled += chunk
+        # publish content hashes of now-complete blocks (prefill only;
+        # shared cached blocks are immutable by construction)
+        full = end // self.pool.block_size
+        if self.mgr.prefix_caching:
+            for b in range(req.registered_blocks, full):
+                self.mgr.register_block(req.request_id, b,
+                                        int(req.block_hashes[b]))
+        req.registered_blocks = max(req.registered_blocks, full)
+        return end == req.prompt_len
+
+    def _prompt_slice(self, req: EngineRequest, start: int, end: int):
+        # vectorized assembly (a per-token python loop here was ~ms per
+        # 4k-token pass and left the GPU idle at steady state)
+        if req._prompt_np is None or len(req._prompt_np) != req.prompt_len:
+            req._prompt_np = np.asarray(req.prompt_tokens, dtype=np.int64)
+        return req._prompt_np[start:end]
+
+    def _prefill_pass(self) -> List[RequestOutput]:
+        selected = self._select_prefill(self.prefill_chunk_tokens)
         if not selected:
             return []
 
@@ -458,32 +531,18 @@ class EngineWorker:
                 base_row = seq_starts[-1] + 0
                 embed_rows.extend(range(base_row, base_row + (e_end - start)))
                 embed_vals.append(req.prefix_embeds[start:e_end])
-            # vectorized assembly (a per-token python loop here was ~ms per
-            # 4k-token pass and left the GPU idle at steady state)
-            if req._prompt_np is None or len(req._prompt_np) != req.prompt_len:
-                req._prompt_np = np.asarray(req.prompt_tokens, dtype=np.int64)
-            ids_np.append(req._prompt_np[start:end])
+            ids_np.append(self._prompt_slice(req, start, end))
             p = np.arange(start, end, dtype=np.int64)
             pos_np.append(p)
             table_np = np.asarray(self.mgr.tables[req.request_id],
                                   dtype=np.int64)
             slots_np.append(table_np[p // bs] * bs + p % bs)
-            self.mgr.set_seq_len(req.request_id, end)
             ctx_lens.append(end)
             tables.append(self.mgr.tables[req.request_id])
             seq_starts.append(seq_starts[-1] + chunk)
-            if end == req.prompt_len:
+            if self._advance_prefill(req, chunk):
                 logit_rows.append(seq_starts[-1] - 1)
                 finishing.append(req)
-            req.computed = end
-            self.total_prefilled += chunk
-            # publish content hashes of now-complete blocks (prefill only;
-            # shared cached blocks are immutable by construction)
-            full = end // bs
-            for b in range(req.registered_blocks, full):
-                self.mgr.register_block(req.request_id, b,
-                                        int(req.block_hashes[b]))
-            req.registered_blocks = max(req.registered_blocks, full)
         input_ids = np.concatenate(ids_np)
         positions = np.concatenate(pos_np)
         slots = np.concatenate(slots_np)
@@ -533,25 +592,17 @@ class EngineWorker:
             if embed_vals else None)
         embedding_reqs = [r for r in finishing if r.is_embedding]
         hidden_or_logits = self.model.forward(
-            batch, self.pool.tensor, embeddings_out=bool(embedding_reqs))
+            batch, self.pool.model_view(),
+            embeddings_out=bool(embedding_reqs))
 
         outputs: List[RequestOutput] = []
-        now = time.time()
         if embedding_reqs:
             # embeddings: mean-pool each finished sequence's chunk rows
             for i, (req, chunk) in enumerate(selected):
-                if req not in embedding_reqs:
-                    continue
-                rows = hidden_or_logits[seq_starts[i]:seq_starts[i + 1]]
-                emb = rows.float().mean(dim=0)
-                outputs.append(RequestOutput(
-                    request_id=req.request_id, new_tokens=[], finished=True,
-                    kind="embedding", embedding=emb.cpu(),
-                    prompt_tokens=req.prompt_len,
-                    e2e_ms=(now - req.arrival_t) * 1e3))
-                self.waiting.remove(req)
-                self.mgr.free(req.request_id)
-                self._by_id.pop(req.request_id, None)
+                if req in embedding_reqs:
+                    outputs.append(self._finish_embedding(
+                        req, hidden_or_logits[seq_starts[i]:
+                                              seq_starts[i + 1]]))
             non_emb = [r for r in finishing if not r.is_embedding]
             if non_emb:
                 # mixed batch: recompute logits for the non-embedding rows
@@ -564,6 +615,17 @@ class EngineWorker:
             if finishing:
                 self._finish_prefills(finishing, hidden_or_logits, outputs)
         return outputs
+
+    def _finish_embedding(self, req: EngineRequest,
+                          rows: torch.Tensor) -> RequestOutput:
+        self.waiting.remove(req)
+        self.mgr.free(req.request_id)
+        self._by_id.pop(req.request_id, None)
+        return RequestOutput(
+            request_id=req.request_id, new_tokens=[], finished=True,
+            kind="embedding", embedding=rows.float().mean(dim=0).cpu(),
+            prompt_tokens=req.prompt_len,
+            e2e_ms=(time.time() - req.arrival_t) * 1e3)
 
     def _finish_prefills(self, finishing, logits, outputs) -> None:
         tokens = self._sample_host(logits, [r.temperature for r in finishing])
@@ -591,29 +653,30 @@ class EngineWorker:
                 if req.slo_ok:
                     self.total_generated_slo += 1
                 self.running.append(req)
-                self.dstate.join(req, self.mgr.tables[req.request_id],
-                                 self.mgr.seq_lens[req.request_id], int(tok))
+                self._join(req, int(tok))
                 outputs.append(RequestOutput(
                     request_id=req.request_id, new_tokens=[int(tok)],
                     ttft_ms=(now - req.arrival_t) * 1e3,
                     cached_tokens=req.cached_tokens))
                 self.total_generated += 1
 
+    def _join(self, req: EngineRequest, last_token: int) -> None:
+        rid = req.request_id
+        self.dstate.join(req, self.mgr.tables[rid], self.mgr.seq_lens[rid],
+                         last_token, self.mgr.slot_of.get(rid, 0))
+
     def release_prefilled(self, request_id: str) -> None:
         """Free a prefill-only sequence after its KV was shipped over xGMI."""
         self.mgr.free(request_id)
 
     # ---- decode ----
-    def _decode_pass(self) -> List[RequestOutput]:
-        """Assemble and launch step N, then collect step N-1's tokens.
-        Membership and finishes are decided from host-side counts, so the
-        launch never waits on token values."""
-        st = self.dstate
-        bs = self.pool.block_size
+    def _select_decode(self):
+        """-> (requests that decode a token this step, requests whose whole
+        generation came from prefill). Allocates the token's slot and puts
+        new blocks into the device tables. Membership and finishes are
+        decided from host-side counts, never from token values."""
         active: List[EngineRequest] = []
-        upd_rows: List[int] = []
-        upd_idx: List[int] = []
-        upd_val: List[int] = []
+        grown: List[str] = []
         done_now: List[EngineRequest] = []
         for req in self.running:
             if len(active) >= self.max_decode_batch:
@@ -623,55 +686,68 @@ class EngineWorker:
                     done_now.append(req)  # all tokens came from prefill
                 continue          # else final token in flight; collect soon
             rid = req.request_id
-            cur = self.mgr.seq_lens[rid]
-            if cur % bs == 0 and len(self.mgr.tables[rid]) <= cur // bs:
-                if not self.mgr.allocate(rid, cur + 1):
-                    continue      # out of KV blocks: stall this sequence
-                upd_rows.append(st.row_of[rid])
-                upd_idx.append(cur // bs)
-                upd_val.append(self.mgr.tables[rid][-1])
-            self.mgr.set_seq_len(rid, cur + 1)
+            if not self._grow_by_one(rid, grown):
+                continue          # out of KV blocks: stall this sequence
             req.inflight += 1
             active.append(req)
+        self._put_new_blocks(grown)
+        return active, done_now
 
-        finals = [self._finalize(r) for r in done_now]
-        if not active:
-            outs = self._collect_pending() + finals
-            # KV exhaustion with every decodable sequence stalled: nothing
-            # will ever free blocks — preempt the youngest running request
-            # (vLLM-style recompute; the prefix cache usually resurrects
-            # its just-freed blocks, so the recompute is mostly free)
-            if self.running and self.mgr.free_blocks == 0:
-                # victim: lowest InferenceObjective priority, youngest last
-                victim = min(reversed(self.running),
-                             key=lambda r: r.priority)
-                po = self._preempt(victim)
-                if po is not None:
-                    outs.append(po)
-            return outs
+    def _grow_by_one(self, rid: str, grown: List[str]) -> bool:
+        """Room for one more token of a decoding sequence."""
+        bs = self.pool.block_size
+        cur = self.mgr.seq_lens[rid]
+        if cur % bs == 0 and len(self.mgr.tables[rid]) <= cur // bs:
+            if not self.mgr.allocate(rid, cur + 1):
+                return False
+            grown.append(rid)
+        self.mgr.set_seq_len(rid, cur + 1)
+        return True
 
-        if upd_rows:
-            st.bt[torch.tensor(upd_rows, dtype=torch.int64, device=self.device),
-                  torch.tensor(upd_idx, dtype=torch.int64, device=self.device)
-                  ] = torch.tensor(upd_val, dtype=torch.int32,
-                                   device=self.device)
+    def _put_new_blocks(self, grown: List[str]) -> None:
+        """Newest block of every grown sequence -> device block tables."""
+        if not grown:
+            return
+        st, tables = self.dstate, self.mgr.tables
 
-        rows_t = st.rows_for([r.request_id for r in active])
-        lens = st.seq_lens.index_select(0, rows_t)
-        new_len = lens + 1
-        pos = new_len - 1                           # int32 positions
+        def dev(vals, dtype):
+            return torch.tensor(vals, dtype=dtype, device=self.device)
+        st.bt[dev([st.row_of[r] for r in grown], torch.int64),
+              dev([len(tables[r]) - 1 for r in grown], torch.int64)] = \
+            dev([tables[r][-1] for r in grown], torch.int32)
+
+    def _decode_rows(self, ids: List[str]):
+        """Device-resident inputs of one more token of every sequence
+        -> (rows, token ids, positions, slots, block tables, new lengths)."""
+        st, bs = self.dstate, self.pool.block_size
+        rows_t = st.rows_for(ids)
+        pos = st.seq_lens.index_select(0, rows_t)   # int32 positions
+        new_len = pos + 1
         bt_rows = st.bt.index_select(0, rows_t)
         blk = bt_rows.gather(
             1, (pos // bs).to(torch.int64).unsqueeze(1)).squeeze(1)
         slot = blk.to(torch.int64) * bs + (pos % bs).to(torch.int64)
         st.seq_lens.index_copy_(0, rows_t, new_len)
-        batch = ForwardBatch(
-            input_ids=st.last_tok.index_select(0, rows_t),
-            positions=pos, slot_mapping=slot, is_decode=True,
-            block_tables=bt_rows, seq_lens=new_len,
-            max_seq_len=max(self.mgr.seq_lens[r.request_id]
-                            for r in active))
-        logits = self.model.forward(batch, self.pool.tensor)
+        return (rows_t, st.last_tok.index_select(0, rows_t), pos, slot,
+                bt_rows, new_len)
+
+    def _nothing_to_decode(self, finals) -> List[RequestOutput]:
+        outs = self._collect_pending() + finals
+        # KV exhaustion with every decodable sequence stalled: nothing
+        # will ever free blocks — preempt the youngest running request
+        # (vLLM-style recompute; the prefix cache usually resurrects
+        # its just-freed blocks, so the recompute is mostly free)
+        if self.running and self.mgr.free_blocks == 0:
+            # victim: lowest InferenceObjective priority, youngest last
+            victim = min(reversed(self.running), key=lambda r: r.priority)
+            po = self._preempt(victim)
+            if po is not None:
+                outs.append(po)
+        return outs
+
+    def _emit_decode(self, active, rows_t, logits) -> List[RequestOutput]:
+        """Sample step N's tokens on the device, collect step N-1's."""
+        st = self.dstate
         any_temp = any(r.temperature > 0 for r in active)
         tok = self._sample_device(logits, rows_t, any_temp)
         st.last_tok.index_copy_(0, rows_t, tok)
@@ -688,7 +764,189 @@ class EngineWorker:
             self._pending = (active, ev, n)
         else:
             self._pending = (active, None, tok)
-        return prev + finals
+        return prev
+
+    def _decode_pass(self) -> List[RequestOutput]:
+        """Assemble and launch step N, then collect step N-1's tokens: the
+        launch never waits on token values."""
+        active, done_now = self._select_decode()
+        finals = [self._finalize(r) for r in done_now]
+        if not active:
+            return self._nothing_to_decode(finals)
+        rows_t, ids, pos, slot, bt_rows, new_len = self._decode_rows(
+            [r.request_id for r in active])
+        batch = ForwardBatch(
+            input_ids=ids, positions=pos, slot_mapping=slot, is_decode=True,
+            block_tables=bt_rows, seq_lens=new_len,
+            max_seq_len=max(self.mgr.seq_lens[r.request_id]
+                            for r in active))
+        logits = self.model.forward(batch, self.pool.model_view())
+        return self._emit_decode(active, rows_t, logits) + finals
+
+    # ---- mixed batches (LayeredRunner) ----
+    def _mixed_batch(self, decode_ids: List[str], portions: List[tuple],
+                     logit_rows: Callable) -> LayeredBatch:
+        """One batch of decoded tokens (device-resident inputs) and portions
+        [(request id, tokens, start)], short ones first. The order of the
+        rows is decode_ids, then `portions` as sorted here in place.
+        logit_rows(first row of every portion) -> rows or None for all."""
+        bs, dev = self.pool.block_size, self.device
+        portions.sort(key=lambda p: len(p[1]) > SHORT)
+        nd, T = len(decode_ids), len(decode_ids)
+        parts = {k: [] for k in ("ids", "pos", "slot", "seq", "meta", "bt")}
+        max_ctx, rows_t = 0, None
+        if nd:
+            rows_t, ids, pos, slot, bt, _ = self._decode_rows(decode_ids)
+            seq = torch.arange(nd, dtype=torch.int32, device=dev)
+            parts["ids"].append(ids)
+            parts["pos"].append(pos)
+            parts["slot"].append(slot)
+            parts["seq"].append(seq)
+            parts["bt"].append(bt)
+            parts["meta"].append(torch.stack(
+                [seq, torch.ones_like(seq), pos,
+                 self.dstate.state_slots.index_select(0, rows_t)], 1))
+            max_ctx = max(self.mgr.seq_lens[r] for r in decode_ids)
+        firsts, long, step_rows, step_seqs = [], [], nd, nd
+        if portions:
+            host = {k: [] for k in ("ids", "pos", "slot", "seq", "meta")}
+            bt = np.zeros((len(portions), self.dstate.max_blocks),
+                          dtype=np.int32)
+            for i, (rid, tokens, start) in enumerate(portions):
+                n, table = len(tokens), self.mgr.tables[rid]
+                p = np.arange(start, start + n, dtype=np.int64)
+                host["ids"].append(np.asarray(tokens, dtype=np.int64))
+                host["pos"].append(p.astype(np.int32))
+                host["slot"].append(np.asarray(table, dtype=np.int64)[p // bs]
+                                    * bs + p % bs)
+                host["seq"].append(np.full(n, nd + i, dtype=np.int32))
+                host["meta"].append(np.array(
+                    [[T, n, start, self.mgr.slot_of.get(rid, 0)]],
+                    dtype=np.int32))
+                bt[i, :len(table)] = table
+                firsts.append(T)
+                if n > SHORT:
+                    long.append(Portion(nd + i, T, n, start, table))
+                else:
+                    step_rows, step_seqs = T + n, nd + i + 1
+                    max_ctx = max(max_ctx, start + n)
+                T += n
+            for k, arrays in host.items():
+                parts[k].append(torch.from_numpy(
+                    np.concatenate(arrays)).to(dev, non_blocking=True))
+            parts["bt"].append(torch.from_numpy(bt).to(dev,
+                                                       non_blocking=True))
+
+        def join(k):
+            return parts[k][0] if len(parts[k]) == 1 else torch.cat(parts[k])
+        rows = logit_rows(firsts)
+        return LayeredBatch(
+            input_ids=join("ids"), positions=join("pos"),
+            slot_mapping=join("slot"), row_seq=join("seq"),
+            seq_meta=join("meta"), block_tables=join("bt"),
+            n_step_seqs=step_seqs, n_step_rows=step_rows,
+            multi_row=T > nd + len(portions), max_ctx=max_ctx, long=long,
+            logit_rows=None if rows is None else torch.tensor(
+                rows, dtype=torch.int64).to(dev, non_blocking=True))
+
+    def _mixed_pass(self, do_prefill: bool) -> List[RequestOutput]:
+        """Portions of waiting prompts and one token of every running
+        request, in one forward."""
+        selected = self._select_prefill(self.prefill_chunk_tokens) \
+            if do_prefill else []
+        active, done_now = self._select_decode()
+        finals = [self._finalize(r) for r in done_now]
+        if not active and not selected:
+            return self._nothing_to_decode(finals)
+        portions, of = [], {}
+        for req, chunk in selected:
+            start = req.computed
+            of[req.request_id] = (
+                req, self._advance_prefill(req, chunk))
+            portions.append((req.request_id, self._prompt_slice(
+                req, start, start + chunk), start))
+        nd = len(active)
+        embed = any(r.is_embedding and last for r, last in of.values())
+
+        def logit_rows(firsts):
+            if embed or not portions:
+                return None
+            return list(range(nd)) + [
+                f + len(p[1]) - 1 for f, p in zip(firsts, portions)
+                if of[p[0]][1]]
+        batch = self._mixed_batch([r.request_id for r in active], portions,
+                                  logit_rows)
+        result = self.model.forward(batch, self.pool.model_view(),
+                                    embeddings_out=embed)
+        outputs: List[RequestOutput] = []
+        finishing, rows, row0 = [], [], nd
+        for rid, tokens, _ in portions:
+            req, last = of[rid]
+            if last and req.is_embedding:
+                outputs.append(self._finish_embedding(
+                    req, result[row0:row0 + len(tokens)]))
+            elif last:
+                finishing.append(req)
+                rows.append(row0 + len(tokens) - 1)
+            row0 += len(tokens)
+        if embed:       # the normed stream came back: project what is needed
+            result = self.model.project(result[list(range(nd)) + rows])
+        if active:
+            outputs.extend(self._emit_decode(
+                active, self.dstate.rows_for([r.request_id for r in active]),
+                result[:nd]))
+        else:
+            outputs.extend(self._collect_pending())
+        if finishing:
+            self._finish_prefills(finishing, result[nd:], outputs)
+        return outputs + finals
+
+    def forward_spans(self, spans: List[TokenSpan],
+                      layers_out: Optional[list] = None) -> torch.Tensor:
+        """Run given tokens instead of sampled ones: one step over all
+        `spans`, from the cache and state that earlier steps left. Requests
+        are admitted at their first span and end with `finish_spans`.
+        -> logits [wanted, vocab], spans in order."""
+        if not self._mixed:
+            raise ValueError("forward_spans needs a mixed-batch model")
+        decode, portions, grown, new = [], [], [], []
+        for s in spans:
+            rid = s.request_id
+            start = self.mgr.seq_lens.get(rid, 0)
+            end = start + len(s.tokens)
+            if not s.tokens or end > self.max_model_len:
+                raise ValueError(f"{rid}: {len(s.tokens)} tokens at {start}")
+            if rid not in self._by_id:
+                self._by_id[rid] = EngineRequest(rid, [], max_tokens=0)
+            if len(s.tokens) == 1 and start > 0:
+                if rid not in self.dstate.row_of:
+                    self._join(self._by_id[rid], 0)
+                if not self._grow_by_one(rid, grown):
+                    raise RuntimeError(f"{rid}: the cache pool is full")
+                decode.append(rid)
+                new.append(s.tokens[0])
+                continue
+            if not self.mgr.allocate(rid, end):
+                raise RuntimeError(f"{rid}: the cache pool is full")
+            self.dstate.leave(rid)
+            self.mgr.set_seq_len(rid, end)
+            portions.append((rid, s.tokens, start))
+        self._put_new_blocks(grown)
+        if decode:
+            self.dstate.last_tok[self.dstate.rows_for(decode)] = torch.tensor(
+                new, dtype=torch.int64, device=self.device)
+
+        def logit_rows(firsts):
+            at = {r: i for i, r in enumerate(decode)}
+            at.update({p[0]: f for f, p in zip(firsts, portions)})
+            return [at[s.request_id] + w for s in spans for w in s.want]
+        batch = self._mixed_batch(decode, portions, logit_rows)
+        return self.model.forward(batch, self.pool.model_view(),
+                                  layers_out=layers_out)
+
+    def finish_spans(self, request_id: str) -> None:
+        """Give back what a request of forward_spans holds."""
+        self.abort(request_id)
 
     def _collect_pending(self) -> List[RequestOutput]:
         if self._pending is None:

@@ -80,6 +80,8 @@ class ForwardBatch:
 
 
 class LlamaRunner:
+    mixed_batches = False       # prefill and decode are passes of their own
+
     def __init__(self, config: ModelConfig, device: torch.device,
                  dtype: torch.dtype = torch.bfloat16, seed: int = 0):
         self.cfg = config

@@ -21,9 +21,11 @@ _SPLIT = re.compile(r"\w+|[^\w\s]")
 class HashTokenizer:
     def __init__(self, vocab_size: int = 128256):
         self.vocab_size = vocab_size
+        self.reserved = min(256, vocab_size // 2)   # low ids, never hashed to
 
     def __call__(self, text: str) -> List[int]:
-        return [rc.xxh64(w.encode("utf-8"), 0) % (self.vocab_size - 256) + 256
+        return [rc.xxh64(w.encode("utf-8"), 0)
+                % (self.vocab_size - self.reserved) + self.reserved
                 for w in _SPLIT.findall(text)]
 
     def decode(self, token_ids: List[int]) -> str:

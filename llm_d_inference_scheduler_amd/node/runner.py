@@ -27,7 +27,8 @@ from ..flowcontrol import (BandConfig, FlowController, FlowRegistry,
                            UtilizationSaturationDetector)
 from ..handlers.parsers import Usage
 from ..metrics import prom
-from ..models.configs import ModelConfig
+from ..models.configs import LayeredConfig
+from ..models.registry import AnyConfig
 from ..parallel.mailbox import Mailbox
 from ..parallel.topology import NodeTopology
 from ..parallel.transfer import KVTransferEngine
@@ -73,7 +74,7 @@ schedulingProfiles:
 
 @dataclass
 class NodeConfig:
-    model: ModelConfig
+    model: AnyConfig
     rank: int = 0
     world_size: int = 1
     topology: str = "mono"
@@ -158,6 +159,11 @@ class NodeRunner:
         self.rank = cfg.rank
         self.topology = NodeTopology.parse(cfg.topology, cfg.world_size)
         self.my_spec = self.topology.ranks[self.rank]
+        if isinstance(cfg.model, LayeredConfig) and \
+                any(r.role != Role.DECODE for r in self.topology.ranks):
+            raise ValueError(f"{cfg.model.name}: this design has no KV "
+                             f"hand-off; use topology mono, not "
+                             f"{cfg.topology}")
         # pipelined (one-step-deep) exchange only when the caller gave the
         # mailbox its own gloo group: pipelining runs the collective on a
         # helper thread, which is only safe if nothing else issues
@@ -188,7 +194,7 @@ class NodeRunner:
         self._emb_pending: Dict[str, torch.Tensor] = {}  # src side
         self._awaiting_embeds: Dict[str, Dict[str, Any]] = {}  # dst side
         transport, peer_pools = self._negotiate_transport(want_ipc)
-        self.transfer = KVTransferEngine(self.engine.pool.tensor, self.rank,
+        self.transfer = KVTransferEngine(self.engine.pool.transfer_view, self.rank,
                                          group=cfg.transfer_group,
                                          transport=transport,
                                          peer_pools=peer_pools)

@@ -1,0 +1,90 @@
+"""Dispatch of the layer-listed designs' ops: `_hip_layered` on GPU tensors
+(required there, no eager fallback), `ref_layered` on CPU tensors."""
+import torch
+
+from . import ref_layered as ref
+
+try:
+    from .. import _hip_layered as _ext
+except ImportError:  # extension not built
+    _ext = None
+
+
+def hip_layered():
+    """The raw extension module. Fail-loud."""
+    if _ext is None:
+        raise RuntimeError(
+            "_hip_layered extension is not built; run "
+            "`python setup.py build_ext --inplace`")
+    return _ext
+
+
+def _impl(t: torch.Tensor):
+    return hip_layered() if t.is_cuda else ref
+
+
+def embed_norm(ids, table, scale, wn, offset, eps):
+    """-> (stream x = table[ids] * scale in 32-bit, its norm)."""
+    return _impl(table).embed_norm(ids, table, scale, wn, offset, eps)
+
+
+def stream_norm(x, y, wb, wn, offset, eps, dtype):
+    """x += rms_norm(y) * (wb + offset), in place (skipped without y);
+    -> rms_norm(x) * (wn + offset) as dtype."""
+    return _impl(x).stream_norm(x, y, wb, wn, offset, eps,
+                                dtype == torch.float32)
+
+
+def gelu_mul(gate_up):
+    """gelu_tanh(gate) * up on packed rows."""
+    return _impl(gate_up).gelu_mul(gate_up)
+
+
+def delta_prep(proj, taps, conv_state, row_seq, seq_meta, multi_row, kv_heads,
+               heads, dim, vdim, q_scale, unit_eps):
+    """Short convolutions, silu and unit norms -> 32-bit q, k, v; the
+    convolution inputs of every sequence move on in conv_state."""
+    return _impl(proj).delta_prep(proj, taps, conv_state, row_seq, seq_meta,
+                                  multi_row, kv_heads, heads, dim, vdim,
+                                  q_scale, unit_eps)
+
+
+def delta_step(q, k, v, proj, beta_col, decay, dt_bias, neg_a, gate, norm_w,
+               state, seq_meta, n_seqs, out, eps):
+    """Token-by-token recurrence of the first n_seqs sequences."""
+    _impl(q).delta_step(q, k, v, proj, beta_col, decay, dt_bias, neg_a, gate,
+                        norm_w, state, seq_meta, n_seqs, out, eps)
+
+
+def latent_prep(proj, wq, wkv, cos_sin, positions, slots, cache, eps):
+    """Norm of the query latent; latent and rotated key part -> cache."""
+    return _impl(proj).latent_prep(proj, wq, wkv, cos_sin, positions, slots,
+                                   cache, eps)
+
+
+def rope_part(q, cos_sin, positions, n_abs):
+    """Rotates the last dims of every head in place; -> the unrotated part
+    of the first n_abs rows, by head."""
+    return _impl(q).rope_part(q, cos_sin, positions, n_abs)
+
+
+def heads_to_rows(src, dst):
+    _impl(src).heads_to_rows(src, dst)
+
+
+def gather_rows(cache, slots):
+    return _impl(cache).gather_rows(cache, slots)
+
+
+def latent_decode(q_lat, q, cache, positions, row_seq, block_tables, window,
+                  scale):
+    """Absorbed attention of single rows over the paged latents."""
+    return _impl(q).attn_rows_paged(q_lat, q, cache, positions, row_seq,
+                                    block_tables, window or 0, scale)
+
+
+def latent_prefill(q, kv, lat, positions, row_seq, base, ctx, rot, window,
+                   scale, out):
+    """Attention of the rows from `base` on over expanded keys and values."""
+    _impl(q).attn_rows_ctx(q, kv, lat, positions, row_seq, base, ctx, rot,
+                           window or 0, scale, out)

@@ -7,6 +7,10 @@ files live inside the package and travel with the repo snapshot:
   * llm_d_inference_scheduler_amd._hip_ops      — gfx950 HIP kernels (torch
     extension, hipcc --offload-arch=gfx950): prefix hash/match, paged KV,
     fused norm/rope/act, GQA decode attention.
+  * llm_d_inference_scheduler_amd._hip_layered  — gfx950 HIP kernels of the
+    layer-listed designs (delta rule, latent attention, 32-bit stream).
+
+LDS_AMD_ONLY=name,... builds only the named modules (e.g. _hip_layered).
 """
 import os
 import sys
@@ -27,6 +31,14 @@ router_core = Pybind11Extension(
     extra_compile_args=["-O3"],
 )
 
+HIP_ARGS = {
+    "cxx": ["-O3"],
+    # packed fp32 instructions stay off: some of their forms have given wrong
+    # results on this hardware
+    "nvcc": ["-O3", "--offload-arch=gfx950", "-std=c++17",
+             "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"],
+}
+
 hip_ops = cpp_extension.CUDAExtension(
     name="llm_d_inference_scheduler_amd._hip_ops",
     sources=[
@@ -38,15 +50,27 @@ hip_ops = cpp_extension.CUDAExtension(
         "csrc/hip/flash_prefill.hip",
         "csrc/hip/flash_prefill_glds.hip",
     ],
-    extra_compile_args={
-        "cxx": ["-O3"],
-        "nvcc": ["-O3", "--offload-arch=gfx950", "-std=c++17"],
-    },
+    extra_compile_args=HIP_ARGS,
+)
+
+hip_layered = cpp_extension.CUDAExtension(
+    name="llm_d_inference_scheduler_amd._hip_layered",
+    sources=[
+        "csrc/hip/layered/ops.hip",
+        "csrc/hip/layered/residual_norm.hip",
+        "csrc/hip/layered/delta_rule.hip",
+        "csrc/hip/layered/latent_attention.hip",
+    ],
+    extra_compile_args=HIP_ARGS,
 )
 
 ext_modules = [router_core]
 if os.environ.get("LDS_AMD_SKIP_HIP", "0") != "1":
-    ext_modules.append(hip_ops)
+    ext_modules += [hip_ops, hip_layered]
+only = os.environ.get("LDS_AMD_ONLY", "")
+if only:
+    ext_modules = [e for e in ext_modules
+                   if e.name.rsplit(".", 1)[-1] in only.split(",")]
 
 setup(
     name="llm_d_inference_scheduler_amd",
