@@ -20,6 +20,14 @@ hipError_t lds_delta_step(int, const float*, const float*, const float*,
                           const float*, const void*, const float*, float*,
                           const int32_t*, void*, int, int, int, int, int,
                           float, hipStream_t);
+int64_t lds_delta_chunk_work(int, int);
+hipError_t lds_delta_chunk(int, const float*, const float*, const float*,
+                           const void*, int64_t, const void*, const float*,
+                           const float*, float*, const int32_t*, int,
+                           const int32_t*, int, float*, float*, int, int, int,
+                           int, hipStream_t);
+hipError_t lds_delta_gate(int, const float*, const void*, const float*, void*,
+                          int64_t, int, float, hipStream_t);
 hipError_t lds_latent_prep(int, const void*, int64_t, const float*,
                            const float*, const float*, const int32_t*,
                            const int64_t*, void*, void*, int, int, int, int,
@@ -215,6 +223,69 @@ void delta_step(Tensor q, Tensor k, Tensor v, Tensor proj, int64_t beta_col,
             "delta_step");
 }
 
+// chunks [n, 2] = first row, tokens (1..64); walk [s, 4] = first row, tokens,
+// slot, first chunk | 1 << 30 for a state that starts at zero. Both on the
+// CPU as well (*_host): the kernels index with them unchecked.
+void delta_chunk(Tensor q, Tensor k, Tensor v, Tensor proj, int64_t beta_col,
+                 Tensor decay, Tensor dt_bias, Tensor neg_a, Tensor state,
+                 Tensor chunks, Tensor walk, Tensor chunks_host,
+                 Tensor walk_host, Tensor ws, Tensor out) {
+  const int f32 = act(proj, "proj");
+  check_delta(q, k, v, proj, beta_col, decay, dt_bias, neg_a, state, f32);
+  const int64_t rows = q.size(0), KH = q.size(1), K = q.size(2);
+  const int64_t H = v.size(1), V = v.size(2);
+  check(chunks, at::kInt, "chunks");
+  check(walk, at::kInt, "walk");
+  const int64_t nc = chunks.size(0), ns = walk.size(0);
+  sized(chunks, {nc, 2}, "chunks");
+  sized(walk, {ns, 4}, "walk");
+  sized(chunks_host, {nc, 2}, "chunks_host");
+  sized(walk_host, {ns, 4}, "walk_host");
+  const auto c = chunks_host.accessor<int32_t, 2>();
+  const auto w = walk_host.accessor<int32_t, 2>();
+  for (int64_t i = 0; i < nc; ++i)
+    TORCH_CHECK(c[i][0] >= 0 && c[i][1] > 0 && c[i][1] <= 64 &&
+                    c[i][0] + c[i][1] <= rows, "chunk ", i);
+  for (int64_t i = 0; i < ns; ++i)
+    TORCH_CHECK(w[i][0] >= 0 && w[i][1] > 0 && w[i][0] + w[i][1] <= rows &&
+                    w[i][2] >= 0 && w[i][2] < state.size(0) &&
+                    (w[i][3] & ((1 << 30) - 1)) + (w[i][1] + 63) / 64 <= nc,
+                "walk ", i);
+  check(ws, at::kFloat, "ws");
+  check(out, at::kFloat, "out");
+  sized(out, {rows, H * V}, "out");
+  const int64_t work = lds_delta_chunk_work((int)K, (int)V);
+  TORCH_CHECK(work > 0 && ws.numel() >= work * nc * H, "ws");
+  const char* beta = (const char*)proj.data_ptr() +
+                     beta_col * proj.element_size();
+  check_hip(lds_delta_chunk(f32, fp(q), fp(k), fp(v), beta, proj.size(1),
+                            decay.data_ptr(), fp(dt_bias), fp(neg_a),
+                            fp(state), ip(chunks), (int)nc, ip(walk), (int)ns,
+                            fp(ws), fp(out), (int)KH, (int)H, (int)K, (int)V,
+                            cur_stream()),
+            "delta_chunk");
+}
+
+// rows [base, rows) of o [rows, H V] -> out
+void delta_gate(Tensor o, Tensor gate, Tensor norm_w, Tensor out,
+                int64_t base, double eps) {
+  check(o, at::kFloat, "o");
+  const int f32 = act(out, "out");
+  same_act(gate, f32, "gate");
+  check(norm_w, at::kFloat, "norm_w");
+  const int64_t rows = o.size(0), HV = o.size(1), V = norm_w.size(0);
+  sized(gate, {rows, HV}, "gate");
+  sized(out, {rows, HV}, "out");
+  TORCH_CHECK(HV % V == 0 && base >= 0 && base <= rows, "delta_gate");
+  const int64_t at = base * HV, es = out.element_size();
+  check_hip(lds_delta_gate(f32, fp(o) + at,
+                           (const char*)gate.data_ptr() + at * es,
+                           fp(norm_w), (char*)out.data_ptr() + at * es,
+                           (rows - base) * (HV / V), (int)V, (float)eps,
+                           cur_stream()),
+            "delta_gate");
+}
+
 Tensor latent_prep(Tensor proj, Tensor wq, OptTensor wkv, Tensor cos_sin,
                    Tensor positions, Tensor slots, OptTensor cache,
                    double eps) {
@@ -367,6 +438,9 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("gelu_mul", &gelu_mul);
   m.def("delta_prep", &delta_prep);
   m.def("delta_step", &delta_step);
+  m.def("delta_chunk_work", &lds_delta_chunk_work);
+  m.def("delta_chunk", &delta_chunk);
+  m.def("delta_gate", &delta_gate);
   m.def("latent_prep", &latent_prep);
   m.def("rope_part", &rope_part);
   m.def("heads_to_rows", &heads_to_rows);

@@ -1,0 +1,90 @@
+"""Prefill and decode throughput of a layer-listed design beside Llama at
+equal layer size (`bench.py --mode layers`): random weights, a stack of a few
+layers, the engine's own steps."""
+import time
+
+import torch
+
+from ..models.configs import ModelConfig, _rururax
+from .worker import EngineRequest, EngineWorker
+
+PATTERN = "ddda" + "ddds"
+VOCAB = 32768
+# name -> width, ff, heads, query rank, latent rank
+SIZES = {"2b": (2048, 8192, 16, 768, 512),
+         "8b": (4096, 14336, 32, 1536, 512),
+         "32b": (5120, 25600, 64, 1536, 512)}
+
+
+def configs(size: str, pattern: str = PATTERN):
+    width, ff, heads, q_rank, kv_rank = SIZES[size]
+    return {
+        "rururax": _rururax(f"rururax-{size}-layers", VOCAB, width, ff,
+                            heads=heads, kv_heads=heads, dim=128,
+                            q_rank=q_rank, kv_rank=kv_rank, window=1024,
+                            pattern=pattern),
+        "llama": ModelConfig(f"llama-{size}-layers", VOCAB, width, ff,
+                             len(pattern), heads, 8, 128)}
+
+
+def measure(cfg, prompts: int, prompt_len: int, batch: int, steps: int,
+            device: str = "cuda:0", dtype=torch.bfloat16) -> dict:
+    """One engine: time prefill steps of prompts x prompt_len tokens, then
+    decode steps of `batch` running requests."""
+    w = EngineWorker(cfg, device, dtype=dtype, kv_budget_bytes=24 << 30,
+                     prefill_chunk_tokens=prompts * prompt_len,
+                     max_decode_batch=batch, prefix_caching=False,
+                     max_model_len=prompt_len + steps + 64)
+    gen = torch.Generator().manual_seed(0)
+    sync = torch.cuda.synchronize if w.device.type == "cuda" else lambda: None
+
+    def add(n, tag, max_tokens):
+        for i in range(n):
+            ids = torch.randint(0, VOCAB, (prompt_len,), generator=gen)
+            w.add_request(EngineRequest(f"{tag}{i}", ids.tolist(),
+                                        max_tokens=max_tokens))
+
+    def prefill(tag):
+        add(prompts, tag, 1)
+        sync()
+        t0 = time.perf_counter()
+        w.step()
+        sync()
+        dt = time.perf_counter() - t0
+        while w.has_work:
+            w.step()
+        return dt
+    prefill("warm")
+    pre = sorted(prefill(f"p{i}-") for i in range(5))[2]
+    add(batch, "d", steps + 40)
+    while len(w.running) < batch:
+        w.step()
+    for _ in range(8):
+        w.step()
+    sync()
+    t0 = time.perf_counter()
+    for _ in range(steps):
+        w.step()
+    sync()
+    dec = time.perf_counter() - t0
+    return {"prefill_tok_s": round(prompts * prompt_len / pre),
+            "prefill_ms": round(pre * 1e3, 3),
+            "decode_tok_s": round(batch * steps / dec),
+            "decode_ms_per_step": round(dec * 1e3 / steps, 3)}
+
+
+def run(sizes, models=("rururax", "llama"), prompts: int = 8,
+        prompt_len: int = 1024, batches=(32, 256), steps: int = 32,
+        pattern: str = PATTERN, device: str = "cuda:0") -> dict:
+    out = {}
+    for size in sizes:
+        cfgs = configs(size, pattern)
+        for b in batches:
+            for name in models:     # both sides in turn
+                out[f"{size}/{name}/batch{b}"] = measure(
+                    cfgs[name], prompts, prompt_len, b, steps, device)
+                if device != "cpu":
+                    torch.cuda.empty_cache()
+                print(f"{size}/{name}/batch{b}",
+                      out[f"{size}/{name}/batch{b}"], flush=True)
+    return out

@@ -826,7 +826,8 @@ class EngineWorker:
                 bt[i, :len(table)] = table
                 firsts.append(T)
                 if n > SHORT:
-                    long.append(Portion(nd + i, T, n, start, table))
+                    long.append(Portion(nd + i, T, n, start, table,
+                                        self.mgr.slot_of.get(rid, 0)))
                 else:
                     step_rows, step_seqs = T + n, nd + i + 1
                     max_ctx = max(max_ctx, start + n)

@@ -26,6 +26,8 @@ from . import rotary
 
 # portions up to this many tokens run like decoded tokens
 SHORT = 8
+CHUNK = 64                  # tokens per chunk of the chunked recurrence
+WORK_BYTES = 160 << 20      # its workspace: stays in the last-level cache
 
 
 @dataclass
@@ -36,6 +38,44 @@ class Portion:
     n: int
     prior: int              # tokens of the sequence before the portion
     table: List[int]        # its blocks
+    slot: int               # its recurrent-state slot
+
+
+@dataclass
+class ChunkGroup:
+    """Chunks of long portions that run with one workspace."""
+    chunks: torch.Tensor        # [n, 2] int32: first row, tokens
+    walk: torch.Tensor          # [s, 4] int32: first row, tokens, state slot,
+    chunks_host: torch.Tensor   # first chunk | 1 << 30 (state starts at zero)
+    walk_host: torch.Tensor
+
+
+def chunk_groups(long: List[Portion], per_group: int,
+                 device: torch.device) -> List[ChunkGroup]:
+    """Cut long portions into chunks, at most `per_group` a group; a portion
+    that does not fit goes on in the next group from its stored state."""
+    groups, chunks, walk = [], [], []
+
+    def close():
+        if chunks:
+            c = torch.tensor(chunks, dtype=torch.int32)
+            w = torch.tensor(walk, dtype=torch.int32)
+            groups.append(ChunkGroup(c.to(device), w.to(device), c, w))
+            chunks.clear()
+            walk.clear()
+    for p in long:
+        at = 0
+        while at < p.n:
+            if len(chunks) == per_group:
+                close()
+            n = min(p.n - at, (per_group - len(chunks)) * CHUNK)
+            fresh = p.prior + at == 0
+            walk.append((p.row0 + at, n, p.slot, len(chunks) | fresh << 30))
+            chunks.extend((p.row0 + a, min(CHUNK, at + n - a))
+                          for a in range(at, at + n, CHUNK))
+            at += n
+    close()
+    return groups
 
 
 @dataclass
@@ -63,11 +103,14 @@ class ChannelDelta:
     """Gated delta rule with one decay per head and key channel."""
 
     def __init__(self, spec: ChannelDeltaSpec, take: Callable, eps: float,
-                 dtype: torch.dtype):
+                 dtype: torch.dtype, device: torch.device):
         self.spec, self.eps = spec, eps
 
         def act(name):
             return take(name).to(dtype)
+        self.work = ops.delta_chunk_work(spec.dim, spec.vdim, device)
+        self.per_group = max(1, WORK_BYTES // max(
+            1, self.work * spec.heads * 4))
         self.w_in = torch.cat([act(n) for n in ("q", "k", "v", "b", "a1",
                                                 "g1")])
         self.beta_col = spec.conv_channels
@@ -91,11 +134,26 @@ class ChannelDelta:
             proj, self.taps, conv_state, batch.row_seq, batch.seq_meta,
             batch.multi_row, s.kv_heads, s.heads, s.dim, s.vdim,
             s.dim ** -0.5, s.unit_eps)
-        out = torch.empty((h.shape[0], s.heads * s.vdim), dtype=h.dtype,
+        T = h.shape[0]
+        out = torch.empty((T, s.heads * s.vdim), dtype=h.dtype,
                           device=h.device)
+        chunked = batch.long and self.work
         ops.delta_step(q, k, v, proj, self.beta_col, decay, self.dt_bias,
                        self.neg_a, gate, self.norm, state, batch.seq_meta,
-                       batch.seq_meta.shape[0], out, self.eps)
+                       batch.n_step_seqs if chunked
+                       else batch.seq_meta.shape[0], out, self.eps)
+        if chunked:
+            o = torch.empty((T, s.heads * s.vdim), dtype=torch.float32,
+                            device=h.device)
+            groups = ctx["chunks", self.per_group]
+            ws = torch.empty(self.work * s.heads * max(
+                len(g.chunks_host) for g in groups), dtype=torch.float32,
+                device=h.device)
+            for g in groups:
+                ops.delta_chunk(q, k, v, proj, self.beta_col, decay,
+                                self.dt_bias, self.neg_a, state, g, ws, o)
+            ops.delta_gate(o, gate, self.norm, out, batch.n_step_rows,
+                           self.eps)
         return linear(out, self.w_o)
 
 
@@ -140,7 +198,7 @@ class LatentAttention:
                                       s.window, s.scale)
             ops.heads_to_rows(torch.bmm(o_lat, self.w_uv), out)
         if n < T:
-            slots, origin = ctx[s.window]
+            slots, origin = ctx["keys", s.window]
             lat = ops.gather_rows(cache, slots)
             kv = linear(lat[:, :s.kv_rank], self.w_ukv)
             ops.latent_prefill(q, kv, lat, batch.positions, batch.row_seq, n,
@@ -167,7 +225,7 @@ class LayeredRunner:
             def mix(name, i=i):
                 return take(f"l{i}.mix.{name}")
             if isinstance(m, ChannelDeltaSpec):
-                self.mixers.append(ChannelDelta(m, mix, eps, dtype))
+                self.mixers.append(ChannelDelta(m, mix, eps, dtype, device))
                 self.kv_layer.append(i)
             else:
                 if m.rot not in tables:
@@ -219,8 +277,13 @@ class LayeredRunner:
         """-> logits of `logit_rows` (or the normed stream of every row).
         layers_out collects copies of the stream after every layer."""
         c = self.cfg
-        ctx = {w: self._context(batch, w, pool.block_size)
-               for w in self.windows} if batch.long else {}
+        ctx = {}            # what layers of equal sizes share
+        if batch.long:
+            for w in self.windows:
+                ctx["keys", w] = self._context(batch, w, pool.block_size)
+            for n in {m.per_group for m in self.mixers
+                      if isinstance(m, ChannelDelta) and m.work}:
+                ctx["chunks", n] = chunk_groups(batch.long, n, self.device)
         pre = [n["norm1"] for n in self.norms] + [self.final_norm]
 
         def norm(y, post, following):

@@ -56,6 +56,26 @@ def delta_step(q, k, v, proj, beta_col, decay, dt_bias, neg_a, gate, norm_w,
                         norm_w, state, seq_meta, n_seqs, out, eps)
 
 
+def delta_chunk_work(dim, vdim, device):
+    """Floats of workspace per (chunk, head); 0 without a chunked form (then
+    delta_step takes every sequence)."""
+    return hip_layered().delta_chunk_work(dim, vdim) \
+        if device.type == "cuda" else 0
+
+
+def delta_chunk(q, k, v, proj, beta_col, decay, dt_bias, neg_a, state, group,
+                ws, out):
+    """Chunked recurrence of the sequences of one ChunkGroup -> 32-bit out."""
+    hip_layered().delta_chunk(q, k, v, proj, beta_col, decay, dt_bias, neg_a,
+                              state, group.chunks, group.walk,
+                              group.chunks_host, group.walk_host, ws, out)
+
+
+def delta_gate(o, gate, norm_w, out, base, eps):
+    """Gated output norm of the rows from `base` on."""
+    hip_layered().delta_gate(o, gate, norm_w, out, base, eps)
+
+
 def latent_prep(proj, wq, wkv, cos_sin, positions, slots, cache, eps):
     """Norm of the query latent; latent and rotated key part -> cache."""
     return _impl(proj).latent_prep(proj, wq, wkv, cos_sin, positions, slots,

@@ -59,6 +59,7 @@ hip_layered = cpp_extension.CUDAExtension(
         "csrc/hip/layered/ops.hip",
         "csrc/hip/layered/residual_norm.hip",
         "csrc/hip/layered/delta_rule.hip",
+        "csrc/hip/layered/delta_chunk.hip",
         "csrc/hip/layered/latent_attention.hip",
     ],
     extra_compile_args=HIP_ARGS,
