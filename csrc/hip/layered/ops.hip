@@ -42,6 +42,17 @@ hipError_t lds_attn_rows(int, const void* const*, const int64_t*, int, int,
                          int, const int32_t*, const int32_t*, int,
                          const int32_t*, int, int, const int32_t*, int, float,
                          void*, int64_t, int64_t, int, int, hipStream_t);
+int lds_latent_decode_ok(int, int, int);
+int lds_latent_decode_parts(int, int, int, int);
+hipError_t lds_latent_decode(const void*, const void*, const void*,
+                             const int32_t*, const int32_t*, const int32_t*,
+                             void*, float*, float*, int, int, int, int, int,
+                             int, int, int, int, float, hipStream_t);
+int lds_latent_prefill_ok(int, int, int, int);
+hipError_t lds_latent_prefill(const void*, const void*, const void*,
+                              const int32_t*, const int32_t*, const int32_t*,
+                              int, void*, int, int, int, int, int, int, float,
+                              hipStream_t);
 }
 
 namespace {
@@ -370,10 +381,11 @@ void check_rows(const Tensor& positions, const Tensor& row_seq, int64_t base,
 }
 
 // q_lat [H, n, R], q [rows, H, D + rot] rotated, cache [NB, BS, R + rot];
-// -> [H, n, R], the first n rows of the batch
-Tensor attn_rows_paged(Tensor q_lat, Tensor q, Tensor cache, Tensor positions,
-                       Tensor row_seq, Tensor block_tables, int64_t window,
-                       double scale) {
+// -> [H, n, R], the first n rows of the batch. bf16 in tiles where the sizes
+// allow it, else (or if `plain`) row by row.
+Tensor latent_decode(Tensor q_lat, Tensor q, Tensor cache, Tensor positions,
+                     Tensor row_seq, Tensor block_tables, int64_t window,
+                     double scale, int64_t max_ctx, bool plain) {
   const int f32 = act(q_lat, "q_lat");
   same_act(q, f32, "q");
   same_act(cache, f32, "cache");
@@ -383,6 +395,26 @@ Tensor attn_rows_paged(Tensor q_lat, Tensor q, Tensor cache, Tensor positions,
   check_rows(positions, row_seq, 0, n);
   TORCH_CHECK(rot >= 0 && Q >= rot && q.size(0) >= n && q.size(1) == H, "q");
   auto out = torch::empty_like(q_lat);
+  if (!f32 && !plain && lds_latent_decode_ok((int)R, (int)rot, (int)Q)) {
+    const int parts = lds_latent_decode_parts((int)n, (int)H, (int)max_ctx,
+                                              (int)window);
+    auto f = q.options().dtype(at::kFloat);
+    Tensor po, ml;
+    if (parts > 1) {
+      po = torch::empty({n, H, parts, R}, f);
+      ml = torch::empty({n, H, parts, 2}, f);
+    }
+    check_hip(lds_latent_decode(
+                  q_lat.data_ptr(), q.data_ptr(), cache.data_ptr(),
+                  ip(positions), ip(row_seq), ip(block_tables),
+                  out.data_ptr(), parts > 1 ? fp(po) : nullptr,
+                  parts > 1 ? fp(ml) : nullptr, (int)n, (int)H, (int)R,
+                  (int)rot, (int)Q, (int)block_tables.size(1),
+                  (int)cache.size(1), (int)window, parts, (float)scale,
+                  cur_stream()),
+              "latent_decode");
+    return out;
+  }
   const int64_t es = q.element_size();
   const char* c = (const char*)cache.data_ptr();
   const void* ptr[5] = {q_lat.data_ptr(),
@@ -399,10 +431,12 @@ Tensor attn_rows_paged(Tensor q_lat, Tensor q, Tensor cache, Tensor positions,
 }
 
 // rows [base, rows): kv [ctx rows, H D + H V], lat [ctx rows, R + rot],
-// ctx [n_seqs, 2] = (first context row, its position); out [rows, H V]
-void attn_rows_ctx(Tensor q, Tensor kv, Tensor lat, Tensor positions,
-                   Tensor row_seq, int64_t base, Tensor ctx, int64_t rot,
-                   int64_t window, double scale, Tensor out) {
+// ctx [n_seqs, 2] = (first context row, its position); out [rows, H V].
+// tiles [n, 2] = (sequence, first row of 128 in its portion).
+void latent_prefill(Tensor q, Tensor kv, Tensor lat, Tensor positions,
+                    Tensor row_seq, int64_t base, Tensor seq_meta, Tensor ctx,
+                    Tensor tiles, int64_t rot, int64_t window, double scale,
+                    Tensor out, bool plain) {
   const int f32 = act(q, "q");
   same_act(kv, f32, "kv");
   same_act(lat, f32, "lat");
@@ -414,6 +448,20 @@ void attn_rows_ctx(Tensor q, Tensor kv, Tensor lat, Tensor positions,
   sized(kv, {lat.size(0), H * (D + V)}, "kv");
   sized(out, {rows, H * V}, "out");
   TORCH_CHECK(D >= 0 && W >= rot && ctx.dim() == 2 && ctx.size(1) == 2, "ctx");
+  if (!f32 && !plain &&
+      lds_latent_prefill_ok((int)D, (int)rot, (int)V, (int)(W - rot))) {
+    check(seq_meta, at::kInt, "seq_meta");
+    check(tiles, at::kInt, "tiles");
+    sized(seq_meta, {ctx.size(0), 4}, "seq_meta");
+    sized(tiles, {tiles.size(0), 2}, "tiles");
+    check_hip(lds_latent_prefill(q.data_ptr(), kv.data_ptr(), lat.data_ptr(),
+                                 ip(seq_meta), ip(ctx), ip(tiles),
+                                 (int)tiles.size(0), out.data_ptr(), (int)H,
+                                 (int)D, (int)rot, (int)V, (int)W,
+                                 (int)window, (float)scale, cur_stream()),
+              "latent_prefill");
+    return;
+  }
   const int64_t es = q.element_size(), KV = kv.size(1);
   const char* qp = (const char*)q.data_ptr() + base * H * Q * es;
   const char* kp = (const char*)kv.data_ptr();
@@ -445,6 +493,6 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("rope_part", &rope_part);
   m.def("heads_to_rows", &heads_to_rows);
   m.def("gather_rows", &gather_rows);
-  m.def("attn_rows_paged", &attn_rows_paged);
-  m.def("attn_rows_ctx", &attn_rows_ctx);
+  m.def("latent_decode", &latent_decode);
+  m.def("latent_prefill", &latent_prefill);
 }

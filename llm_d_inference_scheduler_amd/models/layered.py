@@ -27,6 +27,7 @@ from . import rotary
 # portions up to this many tokens run like decoded tokens
 SHORT = 8
 CHUNK = 64                  # tokens per chunk of the chunked recurrence
+QUERY_TILE = 128            # query rows per workgroup of latent_prefill
 WORK_BYTES = 160 << 20      # its workspace: stays in the last-level cache
 
 
@@ -195,14 +196,15 @@ class LatentAttention:
             q_lat = torch.bmm(q_plain, self.w_uk)
             o_lat = ops.latent_decode(q_lat, q, cache, batch.positions,
                                       batch.row_seq, batch.block_tables,
-                                      s.window, s.scale)
+                                      s.window, s.scale, batch.max_ctx)
             ops.heads_to_rows(torch.bmm(o_lat, self.w_uv), out)
         if n < T:
             slots, origin = ctx["keys", s.window]
             lat = ops.gather_rows(cache, slots)
             kv = linear(lat[:, :s.kv_rank], self.w_ukv)
             ops.latent_prefill(q, kv, lat, batch.positions, batch.row_seq, n,
-                               origin, s.rot_dim, s.window, s.scale, out)
+                               batch.seq_meta, origin, ctx["tiles"],
+                               s.rot_dim, s.window, s.scale, out)
         return linear(out, self.w_o)
 
 
@@ -279,6 +281,11 @@ class LayeredRunner:
         c = self.cfg
         ctx = {}            # what layers of equal sizes share
         if batch.long:
+            if self.windows:
+                ctx["tiles"] = torch.tensor(
+                    [(p.seq, r) for p in batch.long
+                     for r in range(0, p.n, QUERY_TILE)],
+                    dtype=torch.int32).to(self.device)
             for w in self.windows:
                 ctx["keys", w] = self._context(batch, w, pool.block_size)
             for n in {m.per_group for m in self.mixers

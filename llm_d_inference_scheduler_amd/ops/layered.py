@@ -97,14 +97,15 @@ def gather_rows(cache, slots):
 
 
 def latent_decode(q_lat, q, cache, positions, row_seq, block_tables, window,
-                  scale):
+                  scale, max_ctx, plain=False):
     """Absorbed attention of single rows over the paged latents."""
-    return _impl(q).attn_rows_paged(q_lat, q, cache, positions, row_seq,
-                                    block_tables, window or 0, scale)
+    return _impl(q).latent_decode(q_lat, q, cache, positions, row_seq,
+                                  block_tables, window or 0, scale, max_ctx,
+                                  plain)
 
 
-def latent_prefill(q, kv, lat, positions, row_seq, base, ctx, rot, window,
-                   scale, out):
+def latent_prefill(q, kv, lat, positions, row_seq, base, seq_meta, ctx, tiles,
+                   rot, window, scale, out, plain=False):
     """Attention of the rows from `base` on over expanded keys and values."""
-    _impl(q).attn_rows_ctx(q, kv, lat, positions, row_seq, base, ctx, rot,
-                           window or 0, scale, out)
+    _impl(q).latent_prefill(q, kv, lat, positions, row_seq, base, seq_meta,
+                            ctx, tiles, rot, window or 0, scale, out, plain)

@@ -110,8 +110,8 @@ def _attend(s, v, scale):
     return torch.softmax(s * scale, -1) @ v
 
 
-def attn_rows_paged(q_lat, q, cache, positions, row_seq, block_tables, window,
-                    scale):
+def latent_decode(q_lat, q, cache, positions, row_seq, block_tables, window,
+                  scale, max_ctx, plain):
     R, W, bs = q_lat.shape[2], cache.shape[2], cache.shape[1]
     flat = cache.view(-1, W)
     out = torch.empty_like(q_lat)
@@ -126,8 +126,8 @@ def attn_rows_paged(q_lat, q, cache, positions, row_seq, block_tables, window,
     return out
 
 
-def attn_rows_ctx(q, kv, lat, positions, row_seq, base, ctx, rot, window,
-                  scale, out):
+def latent_prefill(q, kv, lat, positions, row_seq, base, seq_meta, ctx, tiles,
+                   rot, window, scale, out, plain):
     rows, H, Q = q.shape
     D, V = Q - rot, out.shape[1] // H
     k = kv[:, :H * D].view(-1, H, D).float()

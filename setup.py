@@ -61,6 +61,8 @@ hip_layered = cpp_extension.CUDAExtension(
         "csrc/hip/layered/delta_rule.hip",
         "csrc/hip/layered/delta_chunk.hip",
         "csrc/hip/layered/latent_attention.hip",
+        "csrc/hip/layered/latent_decode.hip",
+        "csrc/hip/layered/latent_prefill.hip",
     ],
     extra_compile_args=HIP_ARGS,
 )
