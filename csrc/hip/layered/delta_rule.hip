@@ -79,6 +79,75 @@ __global__ __launch_bounds__(NT) void delta_prep_kernel(
   }
 }
 
+// The same for sizes in vectors: a thread owns 8 channels and walks RB rows
+// with the last TAPS - 1 inputs in registers; K / 8 threads (a power of two)
+// share a unit norm. grid (channel blocks, row blocks)
+template <typename T, int TAPS>
+__global__ __launch_bounds__(NT) void delta_prep_vec_kernel(
+    const T* __restrict__ proj, int64_t pstride, const float* __restrict__ taps,
+    T* __restrict__ conv_state, const int32_t* __restrict__ row_seq,
+    const int32_t* __restrict__ seq_meta, float* __restrict__ q,
+    float* __restrict__ k, float* __restrict__ v, int rows, int RB, int KH,
+    int H, int K, int V, float q_scale, float unit_eps) {
+  const int C = 2 * KH * K + H * V, QK = KH * K;
+  const int c = (blockIdx.x * NT + threadIdx.x) * 8;
+  const bool in = c < C;
+  const int cc = in ? c : 0;
+  const bool qk = cc < 2 * QK;
+  float w[TAPS][8], x[TAPS][8];
+#pragma unroll
+  for (int j = 0; j < TAPS; ++j) ldn<8>(taps + (int64_t)j * C + cc, w[j]);
+  const int r0 = blockIdx.y * RB, r1 = min(rows, r0 + RB);
+  for (int row = r0; row < r1; ++row) {
+    const Seq sq = load_seq(seq_meta, row_seq[row]);
+    const int pos = row - sq.row0;
+    T* state = conv_state + (int64_t)sq.slot * (TAPS - 1) * C + cc;
+    if (row == r0 || pos == 0) {
+#pragma unroll
+      for (int j = 0; j < TAPS - 1; ++j) {
+        const int p = pos - (TAPS - 1) + j;
+        if (p >= 0) {
+          ldn<8>(proj + (int64_t)(sq.row0 + p) * pstride + cc, x[j]);
+        } else if (sq.prior > 0) {
+          ldn<8>(state + (int64_t)(TAPS - 1 + p) * C, x[j]);
+        } else {
+#pragma unroll
+          for (int e = 0; e < 8; ++e) x[j][e] = 0.f;
+        }
+      }
+    }
+    ldn<8>(proj + (int64_t)row * pstride + cc, x[TAPS - 1]);
+    if (sq.n == 1 && in) {
+#pragma unroll
+      for (int j = 0; j < TAPS - 1; ++j) stn<8>(state + (int64_t)j * C, x[j + 1]);
+    }
+    float f[8], ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      float a = 0.f;
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) a += w[j][e] * x[j][e];
+      f[e] = a * sigmoid_f(a);
+      ss += f[e] * f[e];
+    }
+    for (int o = K / 16; o > 0; o /= 2) ss += __shfl_xor(ss, o, WAVE);
+    if (qk) {
+      const float m = (cc < QK ? q_scale : 1.f) / sqrtf(ss + unit_eps);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) f[e] *= m;
+    }
+    if (in)
+      stn<8>(cc < QK       ? q + (int64_t)row * QK + cc
+             : cc < 2 * QK ? k + (int64_t)row * QK + cc - QK
+                           : v + (int64_t)row * H * V + cc - 2 * QK,
+             f);
+#pragma unroll
+    for (int j = 0; j < TAPS - 1; ++j)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) x[j][e] = x[j + 1][e];
+  }
+}
+
 // grid (channel blocks, sequences): keep the last n_taps - 1 inputs of every
 // sequence with more than one row (single rows roll in delta_prep)
 template <typename T>
@@ -258,18 +327,34 @@ hipError_t lds_delta_prep(int f32, const void* proj, int64_t pstride,
   int gy = (units + NWV - 1) / NWV;
   if (rows >= 1024 && gy > 4) gy = 4;
   const dim3 grid(rows, gy), cgrid((C + NT - 1) / NT, n_seqs);
+  const bool vec = K % 8 == 0 && V % 8 == 0 && pstride % 8 == 0 &&
+                   K / 8 <= WAVE && (K / 8 & (K / 8 - 1)) == 0 &&
+                   n_taps >= 2 && n_taps <= 4;
+  int rb = 1;       // rows per thread: long walks only with enough of them
+  while (rb < 32 && (int64_t)rows * C / 8 / NT / (2 * rb) >= 2048) rb *= 2;
+  const dim3 vgrid((C / 8 + NT - 1) / NT, (rows + rb - 1) / rb);
+#define VEC(T, TAPS)                                                          \
+  hipLaunchKernelGGL((delta_prep_vec_kernel<T, TAPS>), vgrid, dim3(NT), 0,    \
+                     stream, (const T*)proj, pstride, taps, (T*)conv_state,   \
+                     row_seq, seq_meta, q, k, v, rows, rb, KH, H, K, V,       \
+                     q_scale, unit_eps)
 #define GO(T)                                                                 \
   do {                                                                        \
-    hipLaunchKernelGGL(delta_prep_kernel<T>, grid, dim3(NT), 0, stream,       \
-                       (const T*)proj, pstride, taps, (T*)conv_state,         \
-                       row_seq, seq_meta, q, k, v, KH, H, K, V, n_taps,       \
-                       q_scale, unit_eps);                                    \
+    if (vec && n_taps == 2) VEC(T, 2);                                        \
+    else if (vec && n_taps == 3) VEC(T, 3);                                   \
+    else if (vec) VEC(T, 4);                                                  \
+    else                                                                      \
+      hipLaunchKernelGGL(delta_prep_kernel<T>, grid, dim3(NT), 0, stream,     \
+                         (const T*)proj, pstride, taps, (T*)conv_state,       \
+                         row_seq, seq_meta, q, k, v, KH, H, K, V, n_taps,     \
+                         q_scale, unit_eps);                                  \
     if (multi_row && n_taps > 1)                                              \
       hipLaunchKernelGGL(delta_conv_kernel<T>, cgrid, dim3(NT), 0, stream,    \
                          (const T*)proj, pstride, (T*)conv_state, seq_meta,   \
                          C, n_taps);                                          \
   } while (0)
   if (f32) GO(float); else GO(short);
+#undef VEC
 #undef GO
   HIP_CHECK_LAST();
   return hipSuccess;

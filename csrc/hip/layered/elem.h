@@ -53,11 +53,36 @@ __device__ __forceinline__ void stn(float* p, const float* f) {
   }
 }
 
-__device__ __forceinline__ float sigmoid_f(float x) {
-  return 1.f / (1.f + expf(-x));
+// 1 / x to an ulp or so
+__device__ __forceinline__ float rcp_f(float x) {
+  return __builtin_amdgcn_rcpf(x);
 }
+__device__ __forceinline__ float sigmoid_f(float x) {
+  return rcp_f(1.f + __expf(-x));
+}
+// log(1 + e^x) = max(x, 0) + log(1 + e^-|x|); with e = e^-|x| in (0, 1],
+// log(1 + e) = 2 artanh(s), s = e / (2 + e) <= 1/3: the odd series to s^15
+// leaves less than 1e-8 of the first term, also for small e
 __device__ __forceinline__ float softplus_f(float x) {
-  return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x)));
+  const float e = __expf(-fabsf(x));
+  const float s = e * rcp_f(2.f + e), z = s * s;
+  float p = 1.f / 15.f;
+  p = fmaf(p, z, 1.f / 13.f);
+  p = fmaf(p, z, 1.f / 11.f);
+  p = fmaf(p, z, 1.f / 9.f);
+  p = fmaf(p, z, 1.f / 7.f);
+  p = fmaf(p, z, 1.f / 5.f);
+  p = fmaf(p, z, 1.f / 3.f);
+  p = fmaf(p, z, 1.f);
+  return fmaf(2.f * s, p, fmaxf(x, 0.f));
+}
+
+// Workgroup barrier that orders LDS accesses only: global loads issued before
+// it stay in flight across it (__syncthreads waits for them)
+__device__ __forceinline__ void lds_barrier() {
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "workgroup", "local");
+  __builtin_amdgcn_s_barrier();
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup", "local");
 }
 
 // sum over a block of NW waves; every thread gets it. Two calls in a row

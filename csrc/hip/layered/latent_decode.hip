@@ -89,14 +89,14 @@ __global__ __launch_bounds__(NT) void latent_decode_kernel(
     };
     fetch(t_lo);
     for (int t0 = t_lo; t0 < t_hi; t0 += TB) {
-      __syncthreads();
+      lds_barrier();
 #pragma unroll
       for (int j = 0; j < 2; ++j)
 #pragma unroll
         for (int i = 0; i < NI; ++i)
           if (d0 + i * 64 < WP)
             *(short8*)(kl + (r0 + 32 * j) * LS + d0 + i * 64) = nx[j][i];
-      __syncthreads();
+      lds_barrier();
       if (t0 + TB < t_hi) fetch(t0 + TB);
 
       // scores of this wave's 16 tokens: rows tokens, columns heads
@@ -127,7 +127,7 @@ __global__ __launch_bounds__(NT) void latent_decode_kernel(
         mx = fmaxf(mx, __shfl_xor(mx, 32, WAVE));
         if (grp == 0) red[wave * 16 * HT + a * 16 + col] = mx;
       }
-      __syncthreads();
+      lds_barrier();
       float alpha[HT];
 #pragma unroll
       for (int a = 0; a < HT; ++a) {
@@ -150,7 +150,7 @@ __global__ __launch_bounds__(NT) void latent_decode_kernel(
         sum += __shfl_xor(sum, 32, WAVE);
         if (grp == 0) red[(NW + wave) * 16 * HT + a * 16 + col] = sum;
       }
-      __syncthreads();
+      lds_barrier();
       bf16x8 pf[HT][2];
 #pragma unroll
       for (int a = 0; a < HT; ++a) {

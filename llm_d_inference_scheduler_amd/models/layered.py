@@ -53,29 +53,31 @@ class ChunkGroup:
 
 def chunk_groups(long: List[Portion], per_group: int,
                  device: torch.device) -> List[ChunkGroup]:
-    """Cut long portions into chunks, at most `per_group` a group; a portion
-    that does not fit goes on in the next group from its stored state."""
-    groups, chunks, walk = [], [], []
-
-    def close():
-        if chunks:
-            c = torch.tensor(chunks, dtype=torch.int32)
-            w = torch.tensor(walk, dtype=torch.int32)
-            groups.append(ChunkGroup(c.to(device), w.to(device), c, w))
-            chunks.clear()
-            walk.clear()
-    for p in long:
-        at = 0
-        while at < p.n:
-            if len(chunks) == per_group:
-                close()
-            n = min(p.n - at, (per_group - len(chunks)) * CHUNK)
-            fresh = p.prior + at == 0
-            walk.append((p.row0 + at, n, p.slot, len(chunks) | fresh << 30))
-            chunks.extend((p.row0 + a, min(CHUNK, at + n - a))
-                          for a in range(at, at + n, CHUNK))
-            at += n
-    close()
+    """Cut long portions into chunks, at most `per_group` a group. A group
+    takes a stretch of every portion in turn (they run side by side); the
+    next group goes on from the stored states."""
+    total = sum(-(-p.n // CHUNK) for p in long)
+    per_group = -(-total // -(-total // per_group))     # groups of like size
+    groups = []
+    at = [0] * len(long)
+    while any(a < p.n for a, p in zip(at, long)):
+        left = sum(a < p.n for a, p in zip(at, long))
+        chunks, walk = [], []
+        for i, p in enumerate(long):
+            if at[i] == p.n or len(chunks) == per_group:
+                continue
+            share = max(1, (per_group - len(chunks)) // left)
+            left -= 1
+            n = min(p.n - at[i], share * CHUNK)
+            row = p.row0 + at[i]
+            fresh = p.prior + at[i] == 0
+            walk.append((row, n, p.slot, len(chunks) | fresh << 30))
+            chunks.extend((row + a, min(CHUNK, n - a))
+                          for a in range(0, n, CHUNK))
+            at[i] += n
+        c = torch.tensor(chunks, dtype=torch.int32)
+        w = torch.tensor(walk, dtype=torch.int32)
+        groups.append(ChunkGroup(c.to(device), w.to(device), c, w))
     return groups
 
 
