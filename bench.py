@@ -33,11 +33,16 @@ def parse_args():
     p.add_argument("--steps", type=int, default=200)
     p.add_argument("--warmup", type=int, default=40)
     p.add_argument("--mode", default="mono",
-                   choices=["mono", "pd", "fc", "epd"],
+                   choices=["mono", "pd", "fc", "epd", "layers"],
                    help="mono=prefix-aware DP decode; pd=P/D disagg; "
-                        "fc=flow control at overload; epd=E/P/D multimodal")
+                        "fc=flow control at overload; epd=E/P/D multimodal; "
+                        "layers=prefill and decode of Rururax layers beside "
+                        "Llama layers of equal size (one GPU)")
+    p.add_argument("--layer-sizes", default="2b,8b,32b",
+                   help="sizes of --mode layers, comma-separated")
     p.add_argument("--model", default="llama-3-8b",
-                   help="llama-3-8b | qwen3-32b (the reference regression model)")
+                   help="llama-3-8b | qwen3-32b (the reference regression model) "
+                        "| any registered name or checkpoint folder")
     # the reference's regression harness shape: input 1024 / output 1024
     # (config/manifests/regression-testing/single-workload-regression.yaml)
     p.add_argument("--prompt-len", type=int, default=1024)
@@ -162,6 +167,8 @@ class Workload:
 
 def main():
     args = parse_args()
+    if args.mode == "layers":
+        return layers_main(args)
     wd = float(os.environ.get("LLMD_BENCH_WATCHDOG", "0"))
     if wd > 0:
         # debug: dump all thread stacks and die if the run wedges
@@ -204,8 +211,9 @@ def main():
     else:
         ctrl_group = None
 
+    from llm_d_inference_scheduler_amd.models import registry
     from llm_d_inference_scheduler_amd.models.configs import (
-        LLAMA_3_8B, LLAVA_1_5_7B_TEXT, QWEN3_32B, TINY_LLAMA, TINY_LLAVA)
+        LLAVA_1_5_7B_TEXT, TINY_LLAMA, TINY_LLAVA)
     from llm_d_inference_scheduler_amd.node import NodeConfig, NodeRunner
     from llm_d_inference_scheduler_amd.flowcontrol import BandConfig
     from llm_d_inference_scheduler_amd.api.objectives import InferenceObjective
@@ -215,8 +223,8 @@ def main():
         # world * (weights + KV + activations) fits
         args.kv_gb = min(args.kv_gb, max(16.0, 288.0 / world - 48.0))
 
-    model_cfg = {"llama-3-8b": LLAMA_3_8B,
-                 "qwen3-32b": QWEN3_32B}.get(args.model, TINY_LLAMA)
+    model_cfg = registry.resolve(args.model) if os.path.isdir(args.model) \
+        else registry.MODELS.get(args.model, TINY_LLAMA)
     if args.mode == "epd":
         model_cfg = LLAVA_1_5_7B_TEXT  # BASELINE config 5 multimodal model
         args.model = model_cfg.name
@@ -492,6 +500,32 @@ def main():
     if world > 1:
         dist.barrier()
         dist.destroy_process_group()
+
+
+def layers_main(args):
+    """Throughput of a stack of layers, both designs in turn: one JSON line
+    whose config holds every measurement."""
+    from llm_d_inference_scheduler_amd.engine import layer_bench
+    gpu = torch.cuda.is_available() if args.device is None \
+        else args.device.startswith("cuda")
+    kw = {} if gpu else dict(prompts=2, prompt_len=32, batches=(2,),
+                             device="cpu")
+    sizes = args.layer_sizes.split(",") if gpu else ["tiny"]
+    steps = min(args.steps, 64)
+    rows = layer_bench.run(sizes, steps=steps, **kw)
+    last = [v for k, v in rows.items() if "/rururax/" in k][-1]
+    print(json.dumps({
+        "metric": "Rururax layers: prefill and decode tok/s beside Llama "
+                  "layers of equal size",
+        "value": last["decode_tok_s"], "unit": "tok/s", "n_gpus": 1,
+        "steps": steps, "warmup": 8,
+        "ms_per_step": last["decode_ms_per_step"],
+        "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
+        "dtype": "bf16" if gpu else "fp32",
+        "data": "synthetic prompts, random-init weights",
+        "config": {"model": "rururax layers vs llama layers",
+                   "layers": layer_bench.PATTERN, "parallelism": "dp1",
+                   "results": rows}}), flush=True)
 
 
 def _pctl(xs, p):

@@ -1,6 +1,7 @@
 """Prefill and decode throughput of a layer-listed design beside Llama at
 equal layer size (`bench.py --mode layers`): random weights, a stack of a few
 layers, the engine's own steps."""
+import sys
 import time
 
 import torch
@@ -11,7 +12,8 @@ from .worker import EngineRequest, EngineWorker
 PATTERN = "ddda" + "ddds"
 VOCAB = 32768
 # name -> width, ff, heads, query rank, latent rank
-SIZES = {"2b": (2048, 8192, 16, 768, 512),
+SIZES = {"tiny": (64, 128, 2, 32, 32),      # CPU smoke of the harness
+         "2b": (2048, 8192, 16, 768, 512),
          "8b": (4096, 14336, 32, 1536, 512),
          "32b": (5120, 25600, 64, 1536, 512)}
 
@@ -24,19 +26,22 @@ def configs(size: str, pattern: str = PATTERN):
                             q_rank=q_rank, kv_rank=kv_rank, window=1024,
                             pattern=pattern),
         "llama": ModelConfig(f"llama-{size}-layers", VOCAB, width, ff,
-                             len(pattern), heads, 8, 128)}
+                             len(pattern), heads, min(8, heads), 128)}
 
 
 def measure(cfg, prompts: int, prompt_len: int, batch: int, steps: int,
-            device: str = "cuda:0", dtype=torch.bfloat16) -> dict:
+            device: str = "cuda:0") -> dict:
     """One engine: time prefill steps of prompts x prompt_len tokens, then
     decode steps of `batch` running requests."""
-    w = EngineWorker(cfg, device, dtype=dtype, kv_budget_bytes=24 << 30,
+    gpu = device != "cpu"
+    dtype = torch.bfloat16 if gpu else torch.float32
+    w = EngineWorker(cfg, device, dtype=dtype,
+                     kv_budget_bytes=(24 << 30) if gpu else (64 << 20),
                      prefill_chunk_tokens=prompts * prompt_len,
                      max_decode_batch=batch, prefix_caching=False,
                      max_model_len=prompt_len + steps + 64)
     gen = torch.Generator().manual_seed(0)
-    sync = torch.cuda.synchronize if w.device.type == "cuda" else lambda: None
+    sync = torch.cuda.synchronize if gpu else lambda: None
 
     def add(n, tag, max_tokens):
         for i in range(n):
@@ -86,5 +91,6 @@ def run(sizes, models=("rururax", "llama"), prompts: int = 8,
                 if device != "cpu":
                     torch.cuda.empty_cache()
                 print(f"{size}/{name}/batch{b}",
-                      out[f"{size}/{name}/batch{b}"], flush=True)
+                      out[f"{size}/{name}/batch{b}"], file=sys.stderr,
+                      flush=True)
     return out

@@ -55,3 +55,20 @@ def test_bench_multirank_contract():
     assert r["n_gpus"] == 2
     assert r["config"]["parallelism"] == "dp2"
     assert r["value"] > 0
+
+
+def test_bench_layers_mode():
+    """`--mode layers` prints one JSON line with both designs' numbers."""
+    out = subprocess.run(
+        [sys.executable, "bench.py", "--mode", "layers", "--device", "cpu",
+         "--steps", "2"],
+        cwd=REPO, capture_output=True, text=True, timeout=300)
+    assert out.returncode == 0, out.stderr[-2000:]
+    lines = [l for l in out.stdout.splitlines() if l.startswith("{")]
+    assert len(lines) == 1
+    r = json.loads(lines[0])
+    assert not [k for k in REQUIRED if k not in r]
+    assert set(r["config"]["results"]) == {"tiny/rururax/batch2",
+                                           "tiny/llama/batch2"}
+    for row in r["config"]["results"].values():
+        assert row["prefill_tok_s"] > 0 and row["decode_tok_s"] > 0

@@ -516,6 +516,8 @@ class TestEngineFeaturesGPU:
         assert all(o.completion_tokens == 40 for o in fins.values())
 
 
+@pytest.mark.skip(reason="prefill/decode stream overlap has hung long runs "
+                         "from a cause that is not known; it stays off")
 class TestStreamOverlapGPU:
     def test_overlap_matches_sequential(self):
         """Prefill/decode stream overlap (engine/worker.py step()) is

@@ -1,0 +1,554 @@
+"""Rururax in the engine: every way of cutting and batching a sequence against
+the plain whole-sequence oracle, on the CPU ops and on the HIP kernels."""
+import io
+import itertools
+import json
+import os
+import subprocess
+import sys
+
+import pytest
+import torch
+
+import rururax_models as M
+import rururax_oracle as oracle
+from llm_d_inference_scheduler_amd import trace
+from llm_d_inference_scheduler_amd.engine import EngineRequest, EngineWorker
+from llm_d_inference_scheduler_amd.engine.worker import TokenSpan
+from llm_d_inference_scheduler_amd.models import layered, registry, rururax
+from llm_d_inference_scheduler_amd.models.checkpoint import read_safetensors
+
+ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+GPU = pytest.mark.gpu
+# (device, dtype, tolerance on the rms error relative to the logits' rms: its
+# mean over the tokens; single tokens may have 16 times as much: the norm of a
+# recurrent head's output magnifies the rounding of small ones)
+RUNS = [pytest.param(("cpu", torch.float32, 1e-5), id="cpu-f32"),
+        pytest.param(("cuda:0", torch.float32, 1e-5), id="gpu-f32",
+                     marks=GPU),
+        pytest.param(("cuda:0", torch.bfloat16, 3e-2), id="gpu-bf16",
+                     marks=GPU)]
+CONFIGS = {"odd": M.ODD, "tiled": M.TILED}
+
+
+@pytest.fixture(scope="module")
+def models(tmp_path_factory):
+    """name -> (folder, config, weights), and oracle logits by tokens."""
+    made, known = {}, {}
+
+    def get(name, cfg=None):
+        if name not in made:
+            cfg = cfg or CONFIGS[name]
+            folder, w = M.write_model(
+                tmp_path_factory.mktemp(name), cfg, seed=len(name))
+            made[name] = (folder, cfg, w)
+        return made[name]
+
+    def expect(name, toks):
+        key = (name, tuple(toks))
+        if key not in known:
+            _, cfg, w = made[name]
+            known[key] = oracle.forward(cfg, w, toks)
+        return known[key]
+    get.expect = expect
+    return get
+
+
+def worker(folder, run, blocks=64, slots=4, **kw):
+    device, dtype, _ = run
+    kw.setdefault("max_model_len", 512)
+    return EngineWorker(registry.resolve(folder), device, kv_blocks=blocks,
+                        dtype=dtype, state_slots=slots, **kw)
+
+
+def close(got, want, limit, what=""):
+    got, want = got.double().cpu(), want.double()
+    err = (got - want).pow(2).mean(-1).sqrt() / want.pow(2).mean().sqrt()
+    assert float(err.mean()) < limit and float(err.max()) < 16 * limit, \
+        (what, float(err.mean()), float(err.max()), int(err.argmax()))
+
+
+def tol(name, run):
+    """The small odd sizes average over few channels: noisier in bf16."""
+    return run[2] * (3 if name == "odd" and run[1] == torch.bfloat16 else 1)
+
+
+def feed(w, rid, toks, cuts, every=True):
+    """Run a sequence in portions -> logits of every token (or the last)."""
+    rows, at = [], 0
+    for n in cuts:
+        rows.append(w.forward_spans([TokenSpan(
+            rid, toks[at:at + n], list(range(n)) if every else [n - 1])]))
+        at += n
+    assert at == len(toks)
+    return torch.cat(rows)
+
+
+@pytest.mark.parametrize("run", RUNS)
+@pytest.mark.parametrize("name", ["odd", "tiled"])
+class TestAgainstOracle:
+    def test_whole_and_layers(self, models, name, run):
+        folder, cfg, weights = models(name)
+        toks = M.tokens(cfg, 150)
+        want = []
+        logits = oracle.forward(cfg, weights, toks, want)
+        w = worker(folder, run)
+        got = []
+        out = w.forward_spans([TokenSpan("a", toks, list(range(150)))],
+                              layers_out=got)
+        for i, (a, b) in enumerate(zip(got, want)):
+            close(a, b, tol(name, run), f"layer {i}")
+        close(out, logits, tol(name, run))
+
+    def test_token_by_token(self, models, name, run):
+        folder, cfg, _ = models(name)
+        toks = M.tokens(cfg, 90, 1)
+        w = worker(folder, run)
+        close(feed(w, "a", toks, [1] * 90), models.expect(name, toks),
+              tol(name, run))
+
+    @pytest.mark.parametrize("size", [2, 3, 7, 8, 9, 16, 33, 64, 65])
+    def test_portions(self, models, name, run, size):
+        folder, cfg, _ = models(name)
+        toks = M.tokens(cfg, 140, 2)
+        cuts = [size] * (140 // size) + [140 % size] * (140 % size > 0)
+        w = worker(folder, run)
+        close(feed(w, "a", toks, cuts), models.expect(name, toks), tol(name, run))
+
+    def test_changing_portions_and_long_decoding(self, models, name, run):
+        folder, cfg, _ = models(name)
+        toks = M.tokens(cfg, 260, 3)
+        cuts = [5, 1, 70, 2, 1, 1, 19, 12, 1, 8] + [1] * 140
+        w = worker(folder, run)
+        close(feed(w, "a", toks, cuts), models.expect(name, toks), tol(name, run))
+
+    def test_first_tokens(self, models, name, run):
+        folder, cfg, _ = models(name)
+        w = worker(folder, run)
+        for n, cuts in ((1, [1]), (2, [2]), (3, [1, 2]), (4, [2, 2])):
+            toks = M.tokens(cfg, n, 40 + n)
+            close(feed(w, f"r{n}", toks, cuts), models.expect(name, toks),
+                  tol(name, run))
+            w.finish_spans(f"r{n}")
+
+    def test_mixed_batch_equals_alone(self, models, name, run):
+        """Unequal requests side by side: long and short portions, single
+        tokens, one left out of some steps; pages and slots come from freed
+        requests."""
+        folder, cfg, _ = models(name)
+        w = worker(folder, run, blocks=32)
+        for i in range(5):          # dirty every page and slot first
+            feed(w, f"old{i}", M.tokens(cfg, 100, 60 + i), [37, 63], False)
+            w.finish_spans(f"old{i}")
+        toks = {r: M.tokens(cfg, n, 70 + n) for r, n in
+                (("a", 160), ("b", 45), ("c", 21), ("d", 100), ("e", 75))}
+        plans = {"a": itertools.chain([90, 3, 30], itertools.repeat(1)),
+                 "b": itertools.chain([9, 1, 2], itertools.repeat(1)),
+                 "c": itertools.repeat(1),
+                 "d": itertools.chain([1, 2, 70], itertools.repeat(3)),
+                 "e": itertools.repeat(11)}
+        at, got, live, step = {}, {}, ["a", "b", "c", "d"], 0
+        queue = ["e"]
+        while live:
+            spans = []
+            for r in live:
+                if (step + len(r + "x") + ord(r)) % 5 == 4:
+                    continue        # not in this step
+                n = min(next(plans[r]), len(toks[r]) - at.get(r, 0))
+                lo = at.get(r, 0)
+                spans.append(TokenSpan(r, toks[r][lo:lo + n],
+                                       list(range(n))))
+                at[r] = lo + n
+            if spans:
+                out = w.forward_spans(spans)
+                for s in spans:
+                    got.setdefault(s.request_id, []).append(
+                        out[:len(s.tokens)])
+                    out = out[len(s.tokens):]
+            for r in list(live):
+                if at.get(r) == len(toks[r]):
+                    live.remove(r)
+                    w.finish_spans(r)
+                    if queue:
+                        live.append(queue.pop())
+            step += 1
+        for r, parts in got.items():
+            close(torch.cat(parts), models.expect(name, toks[r]), tol(name, run), r)
+        assert w.mgr.free_blocks == 32 and len(w.mgr._free_slots) == 4
+
+    def test_greedy_generation(self, models, name, run):
+        """Through add_request/step: admission, portions of prompts beside
+        decoding, more requests than slots."""
+        folder, cfg, weights = models(name)
+        w = worker(folder, run, blocks=40, slots=2, prefill_chunk_tokens=24,
+                   prefill_min_tokens=1, max_decode_batch=4)
+        prompts = {f"g{i}": M.tokens(cfg, n, 80 + i)
+                   for i, n in enumerate((30, 1, 57, 12))}
+        for rid, p in prompts.items():
+            w.add_request(EngineRequest(rid, list(p), max_tokens=6))
+        done = {}
+        for _ in range(200):
+            for o in w.step():
+                if o.finished:
+                    done[o.request_id] = o.all_tokens
+            if not w.has_work:
+                break
+        assert set(done) == set(prompts)
+        assert w.mgr.free_blocks == 40 and len(w.mgr._free_slots) == 2
+        margin = 8 * tol(name, run)
+        for rid, p in prompts.items():
+            # every generated token is the oracle's best (or as good as it)
+            logits = oracle.forward(cfg, weights, p + done[rid])
+            for i, t in enumerate(done[rid]):
+                row = logits[len(p) - 1 + i]
+                assert float(row.max() - row[t]) <= \
+                    margin * float(row.pow(2).mean().sqrt()), (rid, i)
+
+
+class TestKeysAndEdges:
+    """A far key that stands out: windows one token off would show."""
+
+    @pytest.mark.parametrize("run", RUNS)
+    @pytest.mark.parametrize("window", [1, 2, 15, 16, 17, 48])
+    def test_window_edges(self, tmp_path, run, window):
+        cfg = M.variant(M.TILED, mask={"size": window})
+        weights = M.random_weights(cfg, 5)
+        for k in weights:
+            if k.endswith(("mix.uq", "mix.uk")):    # peaked scores
+                weights[k] = (weights[k].float() * 2.5).bfloat16()
+        folder, _ = M.write_model(tmp_path / "m", cfg, weights)
+        toks = M.tokens(cfg, 100, 4)
+        want = oracle.forward(cfg, weights, toks)
+        wider = oracle.forward(M.variant(cfg, mask={"size": window + 1}),
+                               weights, toks)
+        shown = (want - wider).pow(2).mean(-1).sqrt() / \
+            want.pow(2).mean().sqrt()
+        assert float(shown.mean()) > 2 * run[2]     # a fault would be seen
+        w = worker(folder, run)
+        for rid, cuts in (("whole", [100]), ("pieces", [41, 2, 20, 37]),
+                          ("decode", [60] + [1] * 40)):
+            close(feed(w, rid, toks, cuts), want, run[2], rid)
+            w.finish_spans(rid)
+
+    @pytest.mark.parametrize("run", RUNS)
+    def test_without_mask(self, tmp_path, run):
+        cfg = M.variant(M.TILED, mask=None)
+        folder, weights = M.write_model(tmp_path / "m", cfg, seed=9)
+        toks = M.tokens(cfg, 120, 6)
+        w = worker(folder, run)
+        close(feed(w, "a", toks, [50, 3, 40] + [1] * 27),
+              oracle.forward(cfg, weights, toks), run[2])
+
+    @pytest.mark.parametrize("run", RUNS)
+    @pytest.mark.parametrize("a_log,bias", [(-6.0, -6.0), (3.0, 2.0)])
+    def test_extreme_decays(self, tmp_path, run, a_log, bias):
+        """States that keep everything, and states that keep nothing."""
+        weights = M.random_weights(M.TILED, 7)
+        for k in weights:
+            if k.endswith("A_log"):
+                weights[k] = (weights[k].float() * 0.3 + a_log).bfloat16()
+            if k.endswith("dt_bias"):
+                weights[k] = (weights[k].float() + 3 + bias).bfloat16()
+        folder, _ = M.write_model(tmp_path / "m", M.TILED, weights)
+        toks = M.tokens(M.TILED, 150, 8)
+        w = worker(folder, run)
+        close(feed(w, "a", toks, [130, 12] + [1] * 8),
+              oracle.forward(M.TILED, weights, toks), run[2])
+
+
+@GPU
+class TestRealisticSizes:
+    """Head sizes of a served model: the widest forms of the kernels."""
+    CFG = {
+        "architecture": "Rururax", "vocab": 128, "width": 256,
+        "embedding": {"scale": 16.0}, "norm": {"eps": 1e-6},
+        "layers": [
+            {"type": "channel_delta", "mlp": {"kind": "dense", "ff": 256},
+             "mixer": {"heads": 3, "kv_heads": 3, "dim": 128, "vdim": 128,
+                       "conv": 4}},
+            {"type": "latent_attention", "mlp": {"kind": "dense", "ff": 256},
+             "mixer": {"heads": 33, "dim": 128, "rot_dim": 64, "vdim": 128,
+                       "q_rank": 192, "kv_rank": 512, "scale": 0.072,
+                       "mask": {"size": 150},
+                       "rot": {"dims": 64, "base": 10000.0,
+                               "scaling": {"factor": 2.0, "original": 128,
+                                           "fast": 32.0, "slow": 1.0}}}},
+            {"type": "latent_attention", "mlp": None,
+             "mixer": {"heads": 16, "dim": 64, "rot_dim": 64, "vdim": 64,
+                       "q_rank": 64, "kv_rank": 512, "scale": 0.09,
+                       "mask": {"size": 400}, "kv_from": 1,
+                       "rot": {"dims": 64, "base": 10000.0,
+                               "scaling": {"factor": 2.0, "original": 128,
+                                           "fast": 32.0, "slow": 1.0}}}},
+        ]}
+
+    @pytest.mark.parametrize("run", RUNS[1:])
+    def test_cuts_and_batches(self, models, run):
+        folder, cfg, _ = models("realistic", self.CFG)
+        w = worker(folder, run, blocks=160, max_model_len=1024)
+        a, b = M.tokens(cfg, 450, 1), M.tokens(cfg, 200, 2)
+        close(feed(w, "a", a, [300, 5, 133] + [1] * 12),
+              models.expect("realistic", a), run[2])
+        out = [w.forward_spans([TokenSpan("b", b[:130], list(range(130)))])]
+        c = M.tokens(cfg, 300, 3)
+        for i in range(70):
+            spans = [TokenSpan("b", [b[130 + i]], [0])]
+            if i == 3:
+                spans.append(TokenSpan("c", c, list(range(300))))
+            r = w.forward_spans(spans)
+            out.append(r[:1])
+            if i == 3:
+                close(r[1:], models.expect("realistic", c), run[2], "c")
+        close(torch.cat(out), models.expect("realistic", b), run[2], "b")
+
+
+class TestChunkGroups:
+    def test_groups_cover_every_portion_in_order(self):
+        P = layered.Portion
+        long = [P(0, 0, 200, 0, [], 3), P(1, 200, 65, 10, [], 1),
+                P(2, 265, 9, 0, [], 0)]
+        for per in (1, 2, 3, 4, 7, 100):
+            done = {p.row0: 0 for p in long}
+            for g in layered.chunk_groups(long, per, torch.device("cpu")):
+                assert len(g.chunks) <= per
+                for row, n, slot, first in g.walk.tolist():
+                    p = max((p for p in long if p.row0 <= row),
+                            key=lambda p: p.row0)
+                    assert row == p.row0 + done[p.row0] and slot == p.slot
+                    fresh = first >> 30
+                    assert fresh == (p.prior + done[p.row0] == 0)
+                    k = first & (1 << 30) - 1
+                    for i in range(0, n, layered.CHUNK):
+                        assert g.chunks[k + i // layered.CHUNK].tolist() == \
+                            [row + i, min(layered.CHUNK, n - i)]
+                    if done[p.row0] + n < p.n:
+                        assert n % layered.CHUNK == 0
+                    done[p.row0] += n
+            assert all(done[p.row0] == p.n for p in long)
+
+
+class TestFramework:
+    def test_reader(self, models):
+        folder, cfg, weights = models("odd")
+        c = registry.resolve(folder)
+        assert (c.vocab_size, c.hidden_size, c.num_layers) == (67, 36, 4)
+        assert c.layers[1].mixer.decay_rank == M.RANKS[0]
+        assert c.layers[1].mixer.gate_rank == M.RANKS[1]
+        assert c.layers[2].mixer.kv_from == 0 and c.layers[2].ff is None
+        assert c.layers[0].mixer.rot.factor is None
+        assert set(rururax.tensor_shapes(c)) == set(weights)
+        assert c.kv_bytes_per_token(2) == 2 * (18 + 4)
+        back = read_safetensors(os.path.join(folder, "model.safetensors"))
+        assert all(torch.equal(back[k], weights[k]) for k in weights)
+
+    @pytest.mark.parametrize("change,text", [
+        (lambda c: c["layers"][0].update(type="other"), "unknown mixer"),
+        (lambda c: c["layers"][1]["mlp"].update(kind="moe"), "unknown mlp"),
+        (lambda c: c["layers"][2]["mixer"].update(kv_from=1), "no latent"),
+        (lambda c: c["layers"][2]["mixer"].update(kv_from=3), "earlier"),
+        (lambda c: c["layers"][2]["mixer"]["rot"].update(base=7.0), "differ"),
+        (lambda c: c["layers"][1]["mixer"].update(kv_heads=4), "multiple"),
+        (lambda c: c.update(architecture="Nope"), "unknown architecture")])
+    def test_bad_configurations(self, tmp_path, change, text):
+        import copy
+        cfg = copy.deepcopy(M.ODD)
+        change(cfg)
+        folder, _ = M.write_model(tmp_path, cfg, M.random_weights(M.ODD))
+        with pytest.raises(ValueError, match=text):
+            registry.resolve(folder)
+
+    def test_missing_tensor(self, tmp_path):
+        w = M.random_weights(M.ODD)
+        del w["l0.mix.uv"]
+        folder, _ = M.write_model(tmp_path, M.ODD, w)
+        with pytest.raises(ValueError, match="l0.mix.uv"):
+            EngineWorker(registry.resolve(folder), "cpu", kv_blocks=8,
+                         dtype=torch.float32)
+        with pytest.raises(ValueError, match="unknown model"):
+            registry.resolve("no-such-model")
+
+    def test_state_slots_gate_admission_and_come_back(self, models):
+        folder, cfg, _ = models("odd")
+        w = worker(folder, ("cpu", torch.float32, 0), blocks=64, slots=1,
+                   prefill_min_tokens=1)
+        for i in range(3):
+            w.add_request(EngineRequest(f"r{i}", M.tokens(cfg, 20, i),
+                                        max_tokens=3))
+        w.step()
+        assert len(w.mgr.slot_of) == 1 and len(w.waiting) == 2
+        for _ in range(60):
+            w.step()
+            if not w.has_work:
+                break
+        assert not w.has_work and w.mgr.slot_of == {}
+
+    def test_preemption_recomputes(self, models):
+        """A pool too small for both: one gives way and starts over."""
+        folder, cfg, weights = models("odd")
+        prompts = {"p": M.tokens(cfg, 40, 1), "q": M.tokens(cfg, 40, 2)}
+        w = worker(folder, ("cpu", torch.float32, 0), blocks=7, slots=2,
+                   prefill_min_tokens=1)
+        for r, p in prompts.items():
+            w.add_request(EngineRequest(r, list(p), max_tokens=20))
+        done = {}
+        for _ in range(300):
+            for o in w.step():
+                if o.finished:
+                    done[o.request_id] = o.all_tokens
+            if not w.has_work:
+                break
+        assert set(done) == set(prompts)
+        for r, p in prompts.items():
+            seq = list(p)
+            for t in done[r]:
+                best = oracle.forward(cfg, weights, seq)[-1]
+                assert float(best.max() - best[t]) < 1e-3
+                seq.append(t)
+
+    def test_no_prefix_reuse_with_recurrent_state(self, models):
+        folder, cfg, _ = models("odd")
+        w = worker(folder, ("cpu", torch.float32, 0))
+        p = M.tokens(cfg, 64, 3)
+        outs = []
+        for r in "ab":
+            w.add_request(EngineRequest(r, list(p), max_tokens=2))
+            for _ in range(20):
+                outs += [o for o in w.step() if o.finished]
+                if not w.has_work:
+                    break
+        assert outs[0].all_tokens == outs[1].all_tokens
+        assert outs[1].cached_tokens == 0
+
+    def test_unsupported_requests_are_refused(self, models):
+        folder, cfg, _ = models("odd")
+        w = worker(folder, ("cpu", torch.float32, 0))
+        w.add_request(EngineRequest("x", [1, 2], prefill_only=True))
+        out = w.step()
+        assert out[0].finished and "unsupported" in out[0].error
+        with pytest.raises(ValueError, match="compute dtype"):
+            EngineWorker(registry.resolve(folder), "cpu", kv_blocks=8,
+                         dtype=torch.float32, kv_cache_dtype="bf16")
+
+    def test_embeddings(self, models):
+        folder, cfg, _ = models("odd")
+        w = worker(folder, ("cpu", torch.float32, 0), prefill_min_tokens=1)
+        w.add_request(EngineRequest("e", M.tokens(cfg, 20), max_tokens=0,
+                                    is_embedding=True))
+        w.add_request(EngineRequest("g", M.tokens(cfg, 9), max_tokens=2))
+        outs = []
+        for _ in range(10):
+            outs += w.step()
+            if not w.has_work:
+                break
+        emb = [o for o in outs if o.kind == "embedding"]
+        assert emb[0].embedding.shape == (36,)
+        assert any(o.finished and o.request_id == "g" for o in outs)
+
+    def test_random_init_is_seeded(self):
+        from llm_d_inference_scheduler_amd.models.configs import TINY_RURURAX
+        outs = []
+        for seed in (3, 3, 4):
+            w = EngineWorker(TINY_RURURAX, "cpu", kv_blocks=16,
+                             dtype=torch.float32, state_slots=1, seed=seed)
+            outs.append(w.forward_spans([TokenSpan("a", [5, 6, 7], [2])]))
+        assert torch.equal(outs[0], outs[1])
+        assert not torch.equal(outs[0], outs[2])
+
+    @pytest.mark.parametrize("run", RUNS)
+    def test_node_generates(self, models, run):
+        """The node's front door: routing, scheduler, engine, completions."""
+        from llm_d_inference_scheduler_amd.node import NodeConfig, NodeRunner
+        from llm_d_inference_scheduler_amd.scheduling.types import LLMRequest
+        folder, cfg, weights = models("tiled")
+        node = NodeRunner(NodeConfig(
+            model=registry.resolve(folder), device=run[0], dtype=run[1],
+            kv_blocks=64, max_decode_batch=4))
+        prompts = {f"n{i}": M.tokens(cfg, 20 + 9 * i, 90 + i)
+                   for i in range(3)}
+        for rid, p in prompts.items():
+            node.submit(LLMRequest(request_id=rid, model="tiled", prompt="",
+                                   prompt_tokens=list(p), max_tokens=5))
+        done = {}
+        for _ in range(100):
+            node.step()
+            for c in node.drain_completions():
+                assert not c.error, c.error
+                done[c.request_id] = c.tokens
+            if len(done) == 3:
+                break
+        node.shutdown()
+        assert set(done) == set(prompts)
+        for rid, p in prompts.items():
+            assert len(done[rid]) == 5
+            logits = oracle.forward(cfg, weights, p + done[rid])
+            for i, t in enumerate(done[rid]):
+                row = logits[len(p) - 1 + i]
+                assert float(row.max() - row[t]) <= \
+                    8 * run[2] * float(row.pow(2).mean().sqrt())
+
+    def test_no_hand_off_topologies(self, models):
+        from llm_d_inference_scheduler_amd.node import NodeConfig, NodeRunner
+        with pytest.raises(ValueError, match="hand-off"):
+            NodeRunner(NodeConfig(model=registry.resolve(models("odd")[0]),
+                                  topology="pd-combined"))
+
+    def test_serve_cli_builds_from_a_folder(self, models):
+        from llm_d_inference_scheduler_amd.server.__main__ import (
+            build_node, parse_args)
+        node = build_node(parse_args(["--model", models("odd")[0],
+                                      "--device", "cpu"]))
+        assert node.engine.model.cfg.hidden_size == 36
+        node.shutdown()
+
+
+class TestTraceRunner:
+    @pytest.mark.parametrize("device,dtype,limit", [
+        ("cpu", "float32", 1e-5),
+        pytest.param("cuda:0", "float32", 1e-5, marks=GPU),
+        pytest.param("cuda:0", "bfloat16", 3e-2, marks=GPU)])
+    def test_replay(self, models, tmp_path, monkeypatch, capsys, device,
+                    dtype, limit):
+        folder, cfg, _ = models("tiled")
+        toks = {"x": M.tokens(cfg, 70, 30), "y": M.tokens(cfg, 50, 31),
+                "z": M.tokens(cfg, 64, 32)}
+        steps = [
+            {"entries": [("x", 40, [0, 39])], "end": []},
+            {"entries": [("x", 1, [0]), ("y", 48, [])], "end": []},
+            {"entries": [("y", 1, [0]), ("x", 29, [28, 3])], "end": ["x"]},
+            {"entries": [("z", 64, [63]), ("y", 1, [0])],
+             "end": ["y", "z"]}]
+        at, lines, want = {}, [], []
+        for n, s in enumerate(steps):
+            entries, rows = [], []
+            for r, k, places in s["entries"]:
+                lo = at.get(r, 0)
+                at[r] = lo + k
+                entries.append({"id": r, "tokens": toks[r][lo:lo + k],
+                                "want": places})
+                rows += [models.expect("tiled", toks[r])[lo + p]
+                         for p in places]
+            lines.append(json.dumps({"step": n, "entries": entries,
+                                     "end": s["end"]}))
+            want.append(rows)
+        # 12 pages: z needs what x gave back
+        argv = ["--model", folder, "--dtype", dtype, "--out", str(tmp_path),
+                "--max-tokens", "192", "--device", device]
+        text = "\n".join(lines) + "\n"
+        if device == "cpu":         # the program itself
+            p = subprocess.run([os.path.join(ROOT, "bin", "trace_run")] + argv,
+                               input=text, capture_output=True, text=True,
+                               timeout=110)
+            assert p.returncode == 0, p.stderr[-2000:]
+            said = p.stdout
+        else:
+            monkeypatch.setattr(sys, "stdin", io.StringIO(text))
+            assert trace.main(argv) == 0
+            said = capsys.readouterr().out
+        assert [x for x in said.splitlines() if x.startswith("done")] \
+            == [f"done {n}" for n in range(4)]
+        for n, rows in enumerate(want):
+            path = tmp_path / f"{n}.f32"
+            raw = torch.frombuffer(bytearray(path.read_bytes()),
+                                   dtype=torch.float32)
+            close(raw.view(len(rows), cfg["vocab"]), torch.stack(rows),
+                  limit)
