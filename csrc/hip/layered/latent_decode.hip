@@ -72,13 +72,21 @@ __global__ __launch_bounds__(NT) void latent_decode_kernel(
     }
     // 8 threads share a token (128 bytes at a time), two tokens per thread
     const int r0 = tid / 8, d0 = tid % 8 * 8;
+    // and their pages one tile further ahead
     short8 nx[2][NI];
+    int page[2];
+    auto find = [&](int t0) {
+#pragma unroll
+      for (int j = 0; j < 2; ++j) {
+        const int t = t0 + r0 + 32 * j;
+        page[j] = t < t_hi ? bt[t / bs] : 0;
+      }
+    };
     auto fetch = [&](int t0) {
 #pragma unroll
       for (int j = 0; j < 2; ++j) {
         const int t = t0 + r0 + 32 * j;
-        const short* src = cache;
-        if (t < t_hi) src += ((int64_t)bt[t / bs] * bs + t % bs) * W;
+        const short* src = cache + ((int64_t)page[j] * bs + t % bs) * W;
 #pragma unroll
         for (int i = 0; i < NI; ++i) {
           const int d = d0 + i * 64;
@@ -87,7 +95,9 @@ __global__ __launch_bounds__(NT) void latent_decode_kernel(
         }
       }
     };
+    find(t_lo);
     fetch(t_lo);
+    find(t_lo + TB);
     for (int t0 = t_lo; t0 < t_hi; t0 += TB) {
       lds_barrier();
 #pragma unroll
@@ -97,12 +107,16 @@ __global__ __launch_bounds__(NT) void latent_decode_kernel(
           if (d0 + i * 64 < WP)
             *(short8*)(kl + (r0 + 32 * j) * LS + d0 + i * 64) = nx[j][i];
       lds_barrier();
-      if (t0 + TB < t_hi) fetch(t0 + TB);
+      if (t0 + TB < t_hi) {
+        fetch(t0 + TB);
+        find(t0 + 2 * TB);
+      }
 
       // scores of this wave's 16 tokens: rows tokens, columns heads
       float4v s[HT];
 #pragma unroll
       for (int a = 0; a < HT; ++a) s[a] = (float4v){0.f, 0.f, 0.f, 0.f};
+#pragma unroll 6
       for (int kk = 0; kk < WP / 32; ++kk) {
         const bf16x8 kf = *(const bf16x8*)(kl + (wave * 16 + col) * LS +
                                            kk * 32 + grp * 8);
@@ -254,8 +268,8 @@ int lds_latent_decode_ok(int R, int rot, int QD) {
 // parts of the context that fill the chip with n rows
 int lds_latent_decode_parts(int n, int H, int max_ctx, int window) {
   const int keys = window > 0 && window < max_ctx ? window : max_ctx;
-  const int groups = n * ((H + 31) / 32);
-  int parts = (256 + groups - 1) / groups;
+  const int groups = n * (H > 16 ? (H + 31) / 32 : 1);
+  int parts = 256 / groups;         // a workgroup has a CU to itself
   if (parts > (keys + 127) / 128) parts = (keys + 127) / 128;
   return parts < 1 ? 1 : parts > 32 ? 32 : parts;
 }
