@@ -2,26 +2,25 @@
 // (bf16): every head of a row reads the same cached token
 // [latent (R) | rotated part], the latent being key part and value at once.
 //
-// One workgroup per (row, 16 or 32 heads, part of the context). Tiles of 64
-// tokens pass through LDS once, for keys and values; the next tile waits in
-// registers. S' = K Q' (wave w owns 16 tokens), softmax across the waves
-// through LDS, O' = V' P' (wave w owns every fourth 16 latent channels; the
-// transposing LDS reads give V'). Memory-bound: the matrix work per token is
-// small beside its bytes.
+// One workgroup per (row, 16 or 32 heads, part of the context), 4 waves per 16
+// heads. Tiles of 64 tokens pass through LDS once, for keys and values; the
+// next tile waits in registers. S' = K Q' (a wave owns 16 tokens and 16 heads),
+// softmax across the waves through LDS, O' = V' P' for all heads (a wave owns
+// every NW-th 16 latent channels; the transposing LDS reads give V').
+// Memory-bound: the matrix work per token is small beside its bytes.
 #include "elem.h"
 
 namespace {
 
-constexpr int NW = 4, NT = NW * WAVE;
 constexpr int TB = 64;          // tokens per tile
 constexpr float NEG = -1e30f;
 constexpr int PS = TB + 8;      // row stride of P (shorts)
 
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
 
-// NTL: 16-channel latent tiles per wave; HT: 16-head tiles
-template <int NTL, int HT>
-__global__ __launch_bounds__(NT) void latent_decode_kernel(
+// RT: latent channels / 64, rounded up; HT: 16-head tiles
+template <int RT, int HT>
+__global__ __launch_bounds__(4 * HT * WAVE) void latent_decode_kernel(
     const short* __restrict__ q_lat,   // [H, n, R]
     const short* __restrict__ q,       // [rows, H, QD], rotated part last
     const short* __restrict__ cache,   // [NB, BS, W]
@@ -31,16 +30,20 @@ __global__ __launch_bounds__(NT) void latent_decode_kernel(
     float* __restrict__ part_ml,       // [n, H, parts, 2]
     int n, int H, int R, int W, int QD, int max_blocks, int bs, int window,
     int parts, float scale_log2) {
-  constexpr int NI = NTL + 1;          // 16-byte pieces per thread and row
+  constexpr int NW = 4 * HT, NT = NW * WAVE;
+  constexpr int NTL = (4 * RT + NW - 1) / NW;  // 16-channel tiles per wave
+  constexpr int NI = RT + 1;           // 16-byte pieces per thread and token
+  constexpr int NJ = 8 / NW;           // tokens per thread and tile
   extern __shared__ short lds[];
   const int WP = (W + 31) / 32 * 32, LS = WP + 8;
   short* kl = lds;                     // [TB][LS]
   short* ql = kl + TB * LS;            // [16 HT][LS]
   short* pl = ql + 16 * HT * LS;       // [16 HT][PS]
-  float* red = (float*)(pl + 16 * HT * PS);   // [2][NW][16 HT]
+  float* red = (float*)(pl + 16 * HT * PS);   // [2][4][16 HT]
   const int row = blockIdx.x, h0 = blockIdx.y * 16 * HT;
   const int tid = threadIdx.x, wave = tid / WAVE, lane = tid % WAVE;
   const int col = lane % 16, grp = lane / 16;
+  const int tw = wave % 4, hw = wave / 4;   // its 16 tokens, its 16 heads
   const int pos = positions[row];
   const int lo = window > 0 ? max(0, pos + 1 - window) : 0;
   const int span = ((pos + 1 - lo + parts - 1) / parts + TB - 1) / TB * TB;
@@ -73,18 +76,18 @@ __global__ __launch_bounds__(NT) void latent_decode_kernel(
     // 8 threads share a token (128 bytes at a time), two tokens per thread
     const int r0 = tid / 8, d0 = tid % 8 * 8;
     // and their pages one tile further ahead
-    short8 nx[2][NI];
-    int page[2];
+    short8 nx[NJ][NI];
+    int page[NJ];
     auto find = [&](int t0) {
 #pragma unroll
-      for (int j = 0; j < 2; ++j) {
+      for (int j = 0; j < NJ; ++j) {
         const int t = t0 + r0 + 32 * j;
         page[j] = t < t_hi ? bt[t / bs] : 0;
       }
     };
     auto fetch = [&](int t0) {
 #pragma unroll
-      for (int j = 0; j < 2; ++j) {
+      for (int j = 0; j < NJ; ++j) {
         const int t = t0 + r0 + 32 * j;
         const short* src = cache + ((int64_t)page[j] * bs + t % bs) * W;
 #pragma unroll
@@ -101,7 +104,7 @@ __global__ __launch_bounds__(NT) void latent_decode_kernel(
     for (int t0 = t_lo; t0 < t_hi; t0 += TB) {
       lds_barrier();
 #pragma unroll
-      for (int j = 0; j < 2; ++j)
+      for (int j = 0; j < NJ; ++j)
 #pragma unroll
         for (int i = 0; i < NI; ++i)
           if (d0 + i * 64 < WP)
@@ -112,57 +115,50 @@ __global__ __launch_bounds__(NT) void latent_decode_kernel(
         find(t0 + 2 * TB);
       }
 
-      // scores of this wave's 16 tokens: rows tokens, columns heads
-      float4v s[HT];
-#pragma unroll
-      for (int a = 0; a < HT; ++a) s[a] = (float4v){0.f, 0.f, 0.f, 0.f};
+      // scores: rows tokens, columns heads
+      float4v sc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll 6
       for (int kk = 0; kk < WP / 32; ++kk) {
-        const bf16x8 kf = *(const bf16x8*)(kl + (wave * 16 + col) * LS +
+        const bf16x8 kf = *(const bf16x8*)(kl + (tw * 16 + col) * LS +
                                            kk * 32 + grp * 8);
-#pragma unroll
-        for (int a = 0; a < HT; ++a) {
-          const bf16x8 qf = *(const bf16x8*)(ql + (a * 16 + col) * LS +
-                                             kk * 32 + grp * 8);
-          s[a] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf, s[a], 0, 0,
-                                                         0);
-        }
+        const bf16x8 qf = *(const bf16x8*)(ql + (hw * 16 + col) * LS +
+                                           kk * 32 + grp * 8);
+        sc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf, sc, 0, 0, 0);
       }
+      float mx = NEG;
 #pragma unroll
-      for (int a = 0; a < HT; ++a) {
-        float mx = NEG;
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int t = t0 + wave * 16 + grp * 4 + r;
-          s[a][r] = t < t_hi ? s[a][r] * scale_log2 : NEG;
-          mx = fmaxf(mx, s[a][r]);
-        }
-        mx = fmaxf(mx, __shfl_xor(mx, 16, WAVE));
-        mx = fmaxf(mx, __shfl_xor(mx, 32, WAVE));
-        if (grp == 0) red[wave * 16 * HT + a * 16 + col] = mx;
+      for (int r = 0; r < 4; ++r) {
+        const int t = t0 + tw * 16 + grp * 4 + r;
+        sc[r] = t < t_hi ? sc[r] * scale_log2 : NEG;
+        mx = fmaxf(mx, sc[r]);
       }
+      mx = fmaxf(mx, __shfl_xor(mx, 16, WAVE));
+      mx = fmaxf(mx, __shfl_xor(mx, 32, WAVE));
+      if (grp == 0) red[(tw * HT + hw) * 16 + col] = mx;
       lds_barrier();
       float alpha[HT];
 #pragma unroll
       for (int a = 0; a < HT; ++a) {
         float mn = m[a];
 #pragma unroll
-        for (int w = 0; w < NW; ++w)
-          mn = fmaxf(mn, red[w * 16 * HT + a * 16 + col]);
+        for (int w = 0; w < 4; ++w)
+          mn = fmaxf(mn, red[(w * HT + a) * 16 + col]);
         alpha[a] = __builtin_amdgcn_exp2f(m[a] - mn);
         m[a] = mn;       // finite: the tile's first token is in range
-        float sum = 0.f, e[4];
+        if (a == hw) {   // wave-uniform
+          float sum = 0.f, e[4];
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          e[r] = __builtin_amdgcn_exp2f(s[a][r] - mn);
-          sum += e[r];
+          for (int r = 0; r < 4; ++r) {
+            e[r] = __builtin_amdgcn_exp2f(sc[r] - mn);
+            sum += e[r];
+          }
+          *(short4v*)(pl + (a * 16 + col) * PS + tw * 16 + grp * 4) =
+              (short4v){f32_to_bf16(e[0]), f32_to_bf16(e[1]),
+                        f32_to_bf16(e[2]), f32_to_bf16(e[3])};
+          sum += __shfl_xor(sum, 16, WAVE);
+          sum += __shfl_xor(sum, 32, WAVE);
+          if (grp == 0) red[((4 + tw) * HT + a) * 16 + col] = sum;
         }
-        *(short4v*)(pl + (a * 16 + col) * PS + wave * 16 + grp * 4) =
-            (short4v){f32_to_bf16(e[0]), f32_to_bf16(e[1]), f32_to_bf16(e[2]),
-                      f32_to_bf16(e[3])};
-        sum += __shfl_xor(sum, 16, WAVE);
-        sum += __shfl_xor(sum, 32, WAVE);
-        if (grp == 0) red[(NW + wave) * 16 * HT + a * 16 + col] = sum;
       }
       lds_barrier();
       bf16x8 pf[HT][2];
@@ -170,8 +166,8 @@ __global__ __launch_bounds__(NT) void latent_decode_kernel(
       for (int a = 0; a < HT; ++a) {
         float sum = 0.f;
 #pragma unroll
-        for (int w = 0; w < NW; ++w)
-          sum += red[(NW + w) * 16 * HT + a * 16 + col];
+        for (int w = 0; w < 4; ++w)
+          sum += red[((4 + w) * HT + a) * 16 + col];
         l[a] = l[a] * alpha[a] + sum;
 #pragma unroll
         for (int ks = 0; ks < 2; ++ks)
@@ -287,8 +283,8 @@ hipError_t lds_latent_decode(const void* q_lat, const void* q,
   const int W = R + rot, LS = (W + 31) / 32 * 32 + 8;
   const int ht = H > 16 ? 2 : 1;
   const size_t lds = (size_t)(TB * LS + 16 * ht * LS + 16 * ht * PS) * 2 +
-                     2 * NW * 16 * ht * sizeof(float);
-  const dim3 grid(n, (H + 16 * ht - 1) / (16 * ht), parts), block(NT);
+                     2 * 4 * 16 * ht * sizeof(float);
+  const dim3 grid(n, (H + 16 * ht - 1) / (16 * ht), parts), block(4 * ht * WAVE);
   const float s2 = scale * 1.4426950408889634f;
 #define GO2(N, HT)                                                            \
   do {                                                                        \
