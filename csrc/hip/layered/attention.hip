@@ -4,8 +4,8 @@
 // pages [n_blocks, block_size, kv_rank + rot_dim]. Rows that come alone (or
 // in short portions) attend to the pages directly, with the key projection
 // absorbed into the query; long portions expand keys and values first
-// (latent_prefill.hip). attn_rows is the plain kernel for either form: any
-// size, bf16 or float.
+// (context_prefill.hip). attn_rows is the plain kernel for either form and for
+// grouped heads: any size, bf16 or float.
 #include "elem.h"
 
 namespace {
@@ -104,14 +104,16 @@ __global__ __launch_bounds__(NT) void gather_rows_kernel(
 }
 
 // Keys and values as the plain kernel sees them: score = qa.ka + qb.kb.
-// Strides in elements; a token is a page slot (block table given) or a
-// context row.
+// Strides in elements; a token is a row of a page (block table given) or a
+// context row. `rep` query heads share a key/value head.
 template <typename T>
 struct View {
   const T *qa, *qb, *ka, *kb, *v;
   int64_t qa_row, qa_head, qb_row, qb_head;
-  int64_t ka_tok, ka_head, kb_tok, v_tok, v_head;
-  int da, db, dv;
+  int64_t ka_tok, ka_head, kb_tok, v_tok, v_head, page;
+  int da, db, dv, rep;
+  int has_sink;
+  float sink;                    // score of a key without a value
 };
 
 // One workgroup per (head, row).
@@ -126,7 +128,7 @@ __global__ __launch_bounds__(NT) void attn_rows_kernel(
     T* __restrict__ out, int64_t o_row, int64_t o_head) {
   extern __shared__ float qv[];  // da + db
   __shared__ float p[NT], redm[NWV], reds[NWV];
-  const int h = blockIdx.x;
+  const int h = blockIdx.x, kvh = h / a.rep;
   const int64_t i = blockIdx.y;       // row of q and out
   const int64_t row = row_base + i;   // row of the batch
   const int seq = row_seq[row];
@@ -136,9 +138,10 @@ __global__ __launch_bounds__(NT) void attn_rows_kernel(
       block_tables ? block_tables + (int64_t)seq * max_blocks : nullptr;
   const int64_t shift =
       bt ? 0 : (int64_t)ctx[2 * seq] - ctx[2 * seq + 1];
-  auto token = [&](int t) -> int64_t {
-    return bt ? (int64_t)bt[t / block_size] * block_size + t % block_size
-              : t + shift;
+  // element offset of a token whose rows are `stride` apart
+  auto at = [&](int t, int64_t stride) -> int64_t {
+    return bt ? bt[t / block_size] * a.page + t % block_size * stride
+              : (t + shift) * stride;
   };
   for (int d = threadIdx.x; d < a.da; d += NT)
     qv[d] = ld(a.qa + i * a.qa_row + h * a.qa_head + d);
@@ -147,15 +150,14 @@ __global__ __launch_bounds__(NT) void attn_rows_kernel(
   float acc[MAXV];
 #pragma unroll
   for (int j = 0; j < MAXV; ++j) acc[j] = 0.f;
-  float m = -INFINITY, l = 0.f;
+  float m = a.has_sink ? a.sink : -INFINITY, l = a.has_sink ? 1.f : 0.f;
   for (int t0 = lo; t0 <= pos; t0 += NT) {
     __syncthreads();
     const int t = t0 + threadIdx.x;
     float s = -INFINITY;
     if (t <= pos) {
-      const int64_t tok = token(t);
-      const T* ka = a.ka + tok * a.ka_tok + h * a.ka_head;
-      const T* kb = a.kb + tok * a.kb_tok;
+      const T* ka = a.ka + at(t, a.ka_tok) + kvh * a.ka_head;
+      const T* kb = a.kb + at(t, a.kb_tok);
       float dot = 0.f;
       for (int d = 0; d < a.da; ++d) dot += qv[d] * ld(ka + d);
       for (int d = 0; d < a.db; ++d) dot += qv[a.da + d] * ld(kb + d);
@@ -167,7 +169,7 @@ __global__ __launch_bounds__(NT) void attn_rows_kernel(
 #pragma unroll
     for (int w = 0; w < NWV; ++w) mx = fmaxf(mx, redm[w]);
     const float mn = fmaxf(m, mx);      // finite: key lo..pos is not empty
-    const float alpha = expf(m - mn);   // 0 at the first tile
+    const float alpha = expf(m - mn);   // 0 at the first tile without a sink
     const float e = t <= pos ? expf(s - mn) : 0.f;
     p[threadIdx.x] = e;
     l = l * alpha + block_sum<NWV>(e, reds);
@@ -179,7 +181,7 @@ __global__ __launch_bounds__(NT) void attn_rows_kernel(
       if (d < a.dv) {
         float o = acc[j] * alpha;
         for (int x = 0; x < n; ++x)
-          o += p[x] * ld(a.v + token(t0 + x) * a.v_tok + h * a.v_head + d);
+          o += p[x] * ld(a.v + at(t0 + x, a.v_tok) + kvh * a.v_head + d);
         acc[j] = o;
       }
     }
@@ -191,18 +193,37 @@ __global__ __launch_bounds__(NT) void attn_rows_kernel(
   }
 }
 
+// rows [.., keys of all heads | values of all heads] from column 0 of kv on
+// -> pages [NB, G, bs, D + V]; U: the unit moved per lane
+template <typename U>
+__global__ __launch_bounds__(NT) void store_heads_kernel(
+    const U* __restrict__ kv, int64_t stride,
+    const int64_t* __restrict__ slots, U* __restrict__ cache, int64_t rows,
+    int G, int bs, int D, int V) {
+  const int W = D + V, width = G * W;
+  const int64_t total = rows * width;
+  for (int64_t i = (int64_t)blockIdx.x * NT + threadIdx.x; i < total;
+       i += (int64_t)gridDim.x * NT) {
+    const int64_t row = i / width, slot = slots[row];
+    const int c = (int)(i % width), g = c / W, d = c % W;
+    cache[((slot / bs * G + g) * bs + slot % bs) * W + d] =
+        kv[row * stride + (d < D ? g * D + d : G * D + g * V + (d - D))];
+  }
+}
+
 template <typename T>
 hipError_t attn_rows_t(const void* const* ptr, const int64_t* stride, int da,
-                       int db, int dv, const int32_t* positions,
-                       const int32_t* row_seq, int row_base,
-                       const int32_t* block_tables, int max_blocks,
-                       int block_size, const int32_t* ctx, int window,
-                       float scale, void* out, int64_t o_row, int64_t o_head,
-                       int rows, int H, hipStream_t stream) {
+                       int db, int dv, int rep, int has_sink, float sink,
+                       const int32_t* positions, const int32_t* row_seq,
+                       int row_base, const int32_t* block_tables,
+                       int max_blocks, int block_size, const int32_t* ctx,
+                       int window, float scale, void* out, int64_t o_row,
+                       int64_t o_head, int rows, int H, hipStream_t stream) {
   View<T> a{(const T*)ptr[0], (const T*)ptr[1], (const T*)ptr[2],
             (const T*)ptr[3], (const T*)ptr[4],
-            stride[0], stride[1], stride[2], stride[3],
-            stride[4], stride[5], stride[6], stride[7], stride[8], da, db, dv};
+            stride[0], stride[1], stride[2], stride[3], stride[4], stride[5],
+            stride[6], stride[7], stride[8], stride[9], da, db, dv, rep,
+            has_sink, sink};
   if (dv > 8 * NT || da + db > 8192) return hipErrorInvalidValue;
   const size_t lds = (size_t)(da + db) * sizeof(float);
   const dim3 block(NT);
@@ -290,9 +311,10 @@ hipError_t lds_gather_rows(const void* cache, const int64_t* slots, void* out,
 }
 
 // ptr: qa, qb, ka, kb, v; stride: qa row/head, qb row/head, ka token/head,
-// kb token, v token/head (elements)
+// kb token, v token/head, page (elements)
 hipError_t lds_attn_rows(int f32, const void* const* ptr,
                          const int64_t* stride, int da, int db, int dv,
+                         int rep, int has_sink, float sink,
                          const int32_t* positions, const int32_t* row_seq,
                          int row_base, const int32_t* block_tables,
                          int max_blocks, int block_size, const int32_t* ctx,
@@ -300,14 +322,33 @@ hipError_t lds_attn_rows(int f32, const void* const* ptr,
                          int64_t o_head, int rows, int H,
                          hipStream_t stream) {
   if (rows == 0) return hipSuccess;
-  return f32 ? attn_rows_t<float>(ptr, stride, da, db, dv, positions, row_seq,
-                                  row_base, block_tables, max_blocks,
-                                  block_size, ctx, window, scale, out, o_row,
-                                  o_head, rows, H, stream)
-             : attn_rows_t<short>(ptr, stride, da, db, dv, positions, row_seq,
-                                  row_base, block_tables, max_blocks,
-                                  block_size, ctx, window, scale, out, o_row,
-                                  o_head, rows, H, stream);
+  auto fn = f32 ? attn_rows_t<float> : attn_rows_t<short>;
+  return fn(ptr, stride, da, db, dv, rep, has_sink, sink, positions, row_seq,
+            row_base, block_tables, max_blocks, block_size, ctx, window, scale,
+            out, o_row, o_head, rows, H, stream);
+}
+
+// es: bytes per element
+hipError_t lds_store_heads(const void* kv, int64_t stride,
+                           const int64_t* slots, void* cache, int64_t rows,
+                           int G, int bs, int D, int V, int es,
+                           hipStream_t stream) {
+  if (rows == 0) return hipSuccess;
+  const int n = 16 / es;      // elements of a 16-byte unit
+  const int u = D % n == 0 && V % n == 0 && stride % n == 0 &&
+                        (uintptr_t)kv % 16 == 0
+                    ? n
+                    : 1;
+  int64_t blocks = (rows * G * (D + V) / u + NT - 1) / NT;
+  if (blocks > 4096) blocks = 4096;
+#define GO(U)                                                                 \
+  hipLaunchKernelGGL(store_heads_kernel<U>, dim3((uint32_t)blocks), dim3(NT), \
+                     0, stream, (const U*)kv, stride / u, slots, (U*)cache,   \
+                     rows, G, bs, D / u, V / u)
+  if (u > 1) GO(short8); else if (es == 4) GO(float); else GO(short);
+#undef GO
+  HIP_CHECK_LAST();
+  return hipSuccess;
 }
 
 }  // extern "C"

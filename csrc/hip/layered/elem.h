@@ -60,6 +60,16 @@ __device__ __forceinline__ float rcp_f(float x) {
 __device__ __forceinline__ float sigmoid_f(float x) {
   return rcp_f(1.f + __expf(-x));
 }
+enum Act { ACT_GELU_TANH, ACT_SILU, ACT_RELU_SQUARED, ACTS };
+__device__ __forceinline__ float activate(int act, float z) {
+  if (act == ACT_RELU_SQUARED) return z > 0.f ? z * z : 0.f;
+  // 0.5 (1 + tanh(a)) = 1 / (1 + exp(-2a))
+  const float a = act == ACT_SILU
+                      ? z
+                      : 2.f * 0.7978845608028654f *
+                            (z + 0.044715f * z * z * z);
+  return z / (1.f + expf(-a));
+}
 // log(1 + e^x) = max(x, 0) + log(1 + e^-|x|); with e = e^-|x| in (0, 1],
 // log(1 + e) = 2 artanh(s), s = e / (2 + e) <= 1/3: the odd series to s^15
 // leaves less than 1e-8 of the first term, also for small e

@@ -1,16 +1,11 @@
 // ops.hip — torch binding of the layered-model kernels (`_hip_layered`).
-// Every shape a kernel's indexing relies on is checked here, on the host.
-#include <torch/extension.h>
-#include <ATen/hip/HIPContext.h>
-#include <ATen/hip/impl/HIPStreamMasqueradingAsCUDA.h>
-
-#include <hip/hip_runtime.h>
+#include "check.h"
 
 extern "C" {
-hipError_t lds_stream_norm(int, float*, const void*, const int64_t*,
-                           const float*, const float*, void*, int64_t, int,
+hipError_t lds_stream_norm(int, int, const void* const*, int64_t, int, int,
                            float, float, float, hipStream_t);
-hipError_t lds_gelu_mul(int, const void*, void*, int64_t, int, hipStream_t);
+hipError_t lds_act(int, int, const void*, void*, int64_t, int, int,
+                   hipStream_t);
 hipError_t lds_delta_prep(int, const void*, int64_t, const float*, void*,
                           const int32_t*, const int32_t*, float*, float*,
                           float*, int, int, int, int, int, int, int, int,
@@ -38,10 +33,6 @@ hipError_t lds_heads_to_rows(int, const void*, void*, int, int, int,
                              hipStream_t);
 hipError_t lds_gather_rows(const void*, const int64_t*, void*, int64_t,
                            int64_t, hipStream_t);
-hipError_t lds_attn_rows(int, const void* const*, const int64_t*, int, int,
-                         int, const int32_t*, const int32_t*, int,
-                         const int32_t*, int, int, const int32_t*, int, float,
-                         void*, int64_t, int64_t, int, int, hipStream_t);
 int lds_latent_decode_ok(int, int, int);
 int lds_latent_decode_parts(int, int, int, int);
 hipError_t lds_latent_decode(const void*, const void*, const void*,
@@ -57,47 +48,6 @@ hipError_t lds_latent_prefill(const void*, const void*, const void*,
 
 namespace {
 
-using torch::Tensor;
-using OptTensor = c10::optional<Tensor>;
-
-hipStream_t cur_stream() {
-  return at::hip::getCurrentHIPStreamMasqueradingAsCUDA().stream();
-}
-
-void check_hip(hipError_t e, const char* what) {
-  TORCH_CHECK(e == hipSuccess, what, ": ", hipGetErrorString(e));
-}
-
-void check(const Tensor& t, at::ScalarType type, const char* name) {
-  TORCH_CHECK(t.is_cuda() && t.is_contiguous(), name,
-              " must be contiguous on the GPU");
-  TORCH_CHECK(t.scalar_type() == type, name, " has type ", t.scalar_type());
-}
-
-void sized(const Tensor& t, std::initializer_list<int64_t> want,
-           const char* name) {
-  TORCH_CHECK(t.sizes() == at::IntArrayRef(want.begin(), want.size()), name,
-              " has sizes ", t.sizes(), ", expected ",
-              at::IntArrayRef(want.begin(), want.size()));
-}
-
-// bf16 or float activations
-int act(const Tensor& t, const char* name) {
-  TORCH_CHECK(t.is_cuda() && t.is_contiguous(), name,
-              " must be contiguous on the GPU");
-  if (t.scalar_type() == at::kFloat) return 1;
-  TORCH_CHECK(t.scalar_type() == at::kBFloat16, name,
-              " must be bf16 or float");
-  return 0;
-}
-
-void same_act(const Tensor& t, int f32, const char* name) {
-  TORCH_CHECK(act(t, name) == f32, name, ": mixed activation types");
-}
-
-float* fp(const Tensor& t) { return t.data_ptr<float>(); }
-int32_t* ip(const Tensor& t) { return t.data_ptr<int32_t>(); }
-
 void check_batch(const Tensor& row_seq, const Tensor& seq_meta, int64_t rows) {
   check(row_seq, at::kInt, "row_seq");
   check(seq_meta, at::kInt, "seq_meta");
@@ -105,55 +55,114 @@ void check_batch(const Tensor& row_seq, const Tensor& seq_meta, int64_t rows) {
   TORCH_CHECK(seq_meta.dim() == 2 && seq_meta.size(1) == 4, "seq_meta");
 }
 
-Tensor stream_norm(Tensor x, OptTensor y, OptTensor wb, Tensor wn,
-                   double offset, double eps, bool f32) {
+enum Mode { EMBED, POST, ADD, LOOP };
+
+void* ptr_or_null(const OptTensor& t) { return t ? t->data_ptr() : nullptr; }
+
+void check_norm(const OptTensor& w, int64_t H, const char* name) {
+  if (!w) return;
+  check(*w, at::kFloat, name);
+  sized(*w, {H}, name);
+}
+
+// without wn the stream itself comes back
+Tensor stream_norm(Tensor x, OptTensor y, OptTensor wb, OptTensor wn,
+                   double offset, double eps, bool f32, OptTensor added) {
   check(x, at::kFloat, "x");
+  TORCH_CHECK(x.dim() == 2, "x");
   const int64_t rows = x.size(0), H = x.size(1);
-  check(wn, at::kFloat, "wn");
-  sized(wn, {H}, "wn");
+  check_norm(wn, H, "wn");
+  check_norm(wb, H, "wb");
   if (y) {
     same_act(*y, f32, "y");
     sized(*y, {rows, H}, "y");
-    TORCH_CHECK(wb.has_value(), "wb goes with y");
-    check(*wb, at::kFloat, "wb");
-    sized(*wb, {H}, "wb");
+  }
+  TORCH_CHECK(y || !wb, "wb goes with y");
+  int64_t n = 0;
+  if (added) {
+    same_act(*added, f32, "rows");
+    n = rows ? added->size(0) / rows : 0;
+    sized(*added, {rows * n, H}, "rows");
   }
   auto h = torch::empty({rows, H},
                         x.options().dtype(f32 ? at::kFloat : at::kBFloat16));
-  check_hip(lds_stream_norm(f32, fp(x), y ? y->data_ptr() : nullptr, nullptr,
-                            y ? fp(*wb) : nullptr, fp(wn), h.data_ptr(), rows,
-                            (int)H, 1.f, (float)offset, (float)eps,
-                            cur_stream()),
+  const void* ptr[12] = {x.data_ptr(), ptr_or_null(y), nullptr, nullptr,
+                         nullptr, ptr_or_null(wb), ptr_or_null(added), nullptr,
+                         nullptr, nullptr, ptr_or_null(wn), h.data_ptr()};
+  check_hip(lds_stream_norm(f32, wb ? POST : ADD, ptr, rows, (int)n, (int)H,
+                            1.f, (float)offset, (float)eps, cur_stream()),
             "stream_norm");
   return h;
 }
 
 std::vector<Tensor> embed_norm(Tensor ids, Tensor table, double scale,
-                               Tensor wn, double offset, double eps) {
+                               OptTensor wn, double offset, double eps,
+                               OptTensor pos, OptTensor positions) {
   check(ids, at::kLong, "ids");
   const int f32 = act(table, "table");
   const int64_t rows = ids.numel(), H = table.size(1);
-  check(wn, at::kFloat, "wn");
-  sized(wn, {H}, "wn");
+  check_norm(wn, H, "wn");
+  if (pos) {
+    check(*pos, at::kFloat, "pos");
+    sized(*pos, {pos->size(0), H}, "pos");
+    TORCH_CHECK(positions.has_value(), "positions go with pos");
+    check(*positions, at::kInt, "positions");
+    sized(*positions, {rows}, "positions");
+  }
   auto x = torch::empty({rows, H}, table.options().dtype(at::kFloat));
   auto h = torch::empty({rows, H}, table.options());
-  check_hip(lds_stream_norm(f32, fp(x), table.data_ptr(),
-                            ids.data_ptr<int64_t>(), nullptr, fp(wn),
-                            h.data_ptr(), rows, (int)H, (float)scale,
+  const void* ptr[12] = {x.data_ptr(), table.data_ptr(), ids.data_ptr(),
+                         ptr_or_null(pos),
+                         pos ? positions->data_ptr() : nullptr, nullptr,
+                         nullptr, nullptr, nullptr, nullptr, ptr_or_null(wn),
+                         h.data_ptr()};
+  check_hip(lds_stream_norm(f32, EMBED, ptr, rows, 0, (int)H, (float)scale,
                             (float)offset, (float)eps, cur_stream()),
             "embed_norm");
   return {x, h};
 }
 
-Tensor gelu_mul(Tensor gate_up) {
-  const int f32 = act(gate_up, "gate_up");
-  TORCH_CHECK(gate_up.dim() == 2 && gate_up.size(1) % 2 == 0, "gate_up");
-  const int64_t rows = gate_up.size(0), I = gate_up.size(1) / 2;
-  auto y = torch::empty({rows, I}, gate_up.options());
-  check_hip(lds_gelu_mul(f32, gate_up.data_ptr(), y.data_ptr(), rows, (int)I,
-                         cur_stream()),
-            "gelu_mul");
+// x = a + b + v
+Tensor loop_norm(Tensor x, Tensor a, Tensor b, Tensor v, OptTensor wn,
+                 double offset, double eps, bool f32) {
+  check(x, at::kFloat, "x");
+  TORCH_CHECK(x.dim() == 2, "x");
+  const int64_t rows = x.size(0), H = x.size(1);
+  for (const Tensor& t : {a, b}) {
+    check(t, at::kFloat, "a, b");
+    sized(t, {rows, H}, "a, b");
+  }
+  check_norm(v, H, "v");
+  check_norm(wn, H, "wn");
+  auto h = torch::empty({rows, H},
+                        x.options().dtype(f32 ? at::kFloat : at::kBFloat16));
+  const void* ptr[12] = {x.data_ptr(), nullptr, nullptr, nullptr, nullptr,
+                         nullptr, nullptr, a.data_ptr(), b.data_ptr(),
+                         v.data_ptr(), ptr_or_null(wn), h.data_ptr()};
+  check_hip(lds_stream_norm(f32, LOOP, ptr, rows, 0, (int)H, 1.f,
+                            (float)offset, (float)eps, cur_stream()),
+            "loop_norm");
+  return h;
+}
+
+Tensor act_rows(const Tensor& x, int64_t I, int gated, int64_t code) {
+  const int f32 = act(x, "x");
+  TORCH_CHECK(code >= 0 && code < 3, "activation ", code);
+  auto y = torch::empty({x.size(0), I}, x.options());
+  check_hip(lds_act(f32, gated, x.data_ptr(), y.data_ptr(), x.size(0), (int)I,
+                    (int)code, cur_stream()),
+            "act");
   return y;
+}
+
+Tensor gated_act(Tensor gate_up, int64_t code) {
+  TORCH_CHECK(gate_up.dim() == 2 && gate_up.size(1) % 2 == 0, "gate_up");
+  return act_rows(gate_up, gate_up.size(1) / 2, 1, code);
+}
+
+Tensor activate(Tensor x, int64_t code) {
+  TORCH_CHECK(x.dim() == 2, "x");
+  return act_rows(x, x.size(1), 0, code);
 }
 
 std::vector<Tensor> delta_prep(Tensor proj, Tensor taps, Tensor conv_state,
@@ -372,14 +381,6 @@ Tensor gather_rows(Tensor cache, Tensor slots) {
   return out;
 }
 
-void check_rows(const Tensor& positions, const Tensor& row_seq, int64_t base,
-                int64_t n) {
-  check(positions, at::kInt, "positions");
-  check(row_seq, at::kInt, "row_seq");
-  TORCH_CHECK(base >= 0 && base + n <= positions.numel() &&
-                  positions.numel() == row_seq.numel(), "batch rows");
-}
-
 // q_lat [H, n, R], q [rows, H, D + rot] rotated, cache [NB, BS, R + rot];
 // -> [H, n, R], the first n rows of the batch. bf16 in tiles where the sizes
 // allow it, else (or if `plain`) row by row.
@@ -420,8 +421,10 @@ Tensor latent_decode(Tensor q_lat, Tensor q, Tensor cache, Tensor positions,
   const void* ptr[5] = {q_lat.data_ptr(),
                         (const char*)q.data_ptr() + (Q - rot) * es, c,
                         c + R * es, c};
-  const int64_t stride[9] = {R, n * R, H * Q, Q, W, 0, W, W, 0};
-  check_hip(lds_attn_rows(f32, ptr, stride, (int)R, (int)rot, (int)R,
+  const int64_t stride[10] = {R, n * R, H * Q, Q, W, 0, W, W, 0,
+                              cache.size(1) * W};
+  check_hip(lds_attn_rows(f32, ptr, stride, (int)R, (int)rot, (int)R, (int)H,
+                          0, 0.f,
                           ip(positions), ip(row_seq), 0, ip(block_tables),
                           (int)block_tables.size(1), (int)cache.size(1),
                           nullptr, (int)window, (float)scale, out.data_ptr(),
@@ -468,8 +471,9 @@ void latent_prefill(Tensor q, Tensor kv, Tensor lat, Tensor positions,
   const void* ptr[5] = {qp, qp + D * es, kp,
                         (const char*)lat.data_ptr() + (W - rot) * es,
                         kp + H * D * es};
-  const int64_t stride[9] = {H * Q, Q, H * Q, Q, KV, D, W, KV, V};
-  check_hip(lds_attn_rows(f32, ptr, stride, (int)D, (int)rot, (int)V,
+  const int64_t stride[10] = {H * Q, Q, H * Q, Q, KV, D, W, KV, V, 0};
+  check_hip(lds_attn_rows(f32, ptr, stride, (int)D, (int)rot, (int)V, 1, 0,
+                          0.f,
                           ip(positions), ip(row_seq), (int)base, nullptr, 0, 1,
                           ip(ctx), (int)window, (float)scale,
                           (char*)out.data_ptr() + base * H * V * es, H * V, V,
@@ -483,7 +487,9 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.doc() = "gfx950 kernels of the layer-listed designs";
   m.def("stream_norm", &stream_norm);
   m.def("embed_norm", &embed_norm);
-  m.def("gelu_mul", &gelu_mul);
+  m.def("loop_norm", &loop_norm);
+  m.def("gated_act", &gated_act);
+  m.def("activate", &activate);
   m.def("delta_prep", &delta_prep);
   m.def("delta_step", &delta_step);
   m.def("delta_chunk_work", &lds_delta_chunk_work);
@@ -495,4 +501,5 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("gather_rows", &gather_rows);
   m.def("latent_decode", &latent_decode);
   m.def("latent_prefill", &latent_prefill);
+  bind_grouped(m);
 }

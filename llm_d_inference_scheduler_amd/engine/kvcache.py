@@ -107,11 +107,13 @@ class KVPool:
 
 
 class LayeredPool:
-    """Cache of a layer-listed design. A latent-attention layer that owns its
-    latents has pages [num_blocks, block_size, kv_rank + rot_dim] (layers
-    that attend to another layer's latents have none); a recurrent layer has
-    one slot per live sequence: convolution inputs [slots, taps - 1,
-    channels] and the matrix state [slots, heads, dim, vdim] in 32-bit.
+    """Cache of a layer-listed design, one entry per run of a layer (a looped
+    layer has one for each pass). Attention has pages: [num_blocks,
+    block_size, kv_rank + rot_dim] for latents, [num_blocks, kv_heads,
+    block_size, dim + vdim] for grouped heads, none for a layer that attends
+    to another one's. A recurrent layer has one slot per live sequence:
+    convolution inputs [slots, taps - 1, channels] and the matrix state
+    [slots, heads, dim, vdim] in 32-bit.
 
     Slots are never cleared: the kernels start a sequence without earlier
     tokens from zero."""
@@ -127,8 +129,8 @@ class LayeredPool:
         self.state_slots = state_slots if config.has_recurrent_state else 0
         self.ipc_backed = False
         self.layers: List[object] = []
-        for layer in config.layers:
-            m = layer.mixer
+        for run in config.runs:
+            m = config.layers[run.layer].mixer
             if isinstance(m, ChannelDeltaSpec):
                 state, conv = m.state_shapes
                 self.layers.append((
@@ -138,7 +140,7 @@ class LayeredPool:
                                 device=device)))
             elif m.cache_width:
                 self.layers.append(torch.zeros(
-                    (num_blocks, block_size, m.cache_width), dtype=dtype,
+                    (num_blocks,) + m.page_shape(block_size), dtype=dtype,
                     device=device))
             else:
                 self.layers.append(None)

@@ -207,6 +207,9 @@ class EngineWorker:
         self.prefill_min_tokens = prefill_min_tokens
         self.prefill_max_delay_ms = prefill_max_delay_ms
         self.max_decode_batch = max_decode_batch
+        if getattr(config, "learned_positions", False):
+            # there is no vector for a position past the table
+            max_model_len = min(max_model_len, config.max_position)
         self.max_model_len = max_model_len
         self.ttft_slo_ms = ttft_slo_ms
         cache_dtype = {"auto": dtype, "bf16": torch.bfloat16,

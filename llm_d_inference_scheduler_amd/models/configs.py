@@ -112,6 +112,11 @@ class ChannelDeltaSpec:
         return 2 * self.kv_heads * self.dim + self.heads * self.vdim
 
     @property
+    def cache_width(self) -> int:
+        """Cached values per token: none, the state has a fixed size."""
+        return 0
+
+    @property
     def state_shapes(self) -> Tuple[Tuple[int, ...], Tuple[int, ...]]:
         """Per sequence: matrix state (32-bit), convolution inputs."""
         return ((self.heads, self.dim, self.vdim),
@@ -137,14 +142,77 @@ class LatentAttentionSpec:
         """Cached values per token (0: the layer owns no cache)."""
         return 0 if self.kv_from is not None else self.kv_rank + self.rot_dim
 
+    def page_shape(self, block_size: int) -> Tuple[int, ...]:
+        return block_size, self.cache_width
 
-MixerSpec = Union[ChannelDeltaSpec, LatentAttentionSpec]
+
+@dataclass(frozen=True)
+class GroupedAttentionSpec:
+    """Causal attention, query heads in groups that share a key/value head;
+    positions do not enter the scores."""
+    heads: int
+    kv_heads: int
+    dim: int                        # query/key size per head
+    vdim: int
+    scale: float
+    sink: Optional[float] = None    # score of an extra key without a value
+
+    @property
+    def cache_width(self) -> int:
+        return self.kv_heads * (self.dim + self.vdim)
+
+    def page_shape(self, block_size: int) -> Tuple[int, ...]:
+        """A head's tokens of a page lie together, rows [key | value]."""
+        return self.kv_heads, block_size, self.dim + self.vdim
+
+
+MixerSpec = Union[ChannelDeltaSpec, LatentAttentionSpec, GroupedAttentionSpec]
+
+
+@dataclass(frozen=True)
+class GatedSpec:
+    """Feed-forward down(act(gate h) * up h)."""
+    ff: int
+    act: str = "gelu_tanh"
+
+
+@dataclass(frozen=True)
+class ExpertsSpec:
+    """Feed-forward of experts down(act(up h)). A token goes to the `top`
+    experts with the largest scores sigmoid(router h); the score multiplies
+    the expert's input. A shared expert takes every token."""
+    experts: int
+    top: int
+    ff: int                         # inner size of one expert
+    shared_ff: Optional[int] = None     # of the shared one (None: has none)
+    act: str = "relu_squared"
+
+
+FeedForwardSpec = Union[GatedSpec, ExpertsSpec]
 
 
 @dataclass(frozen=True)
 class LayerSpec:
     mixer: MixerSpec
-    ff: Optional[int] = None        # gated MLP size (None: no feed-forward)
+    ff: Optional[FeedForwardSpec] = None    # None: no feed-forward
+
+
+@dataclass(frozen=True)
+class LoopSpec:
+    """Layers start .. stop-1 run `times` times in a row with the same
+    weights. Ahead of each pass the stream is mixed with the embedding output
+    and gets a vector of that pass."""
+    start: int
+    stop: int
+    times: int
+
+
+@dataclass(frozen=True)
+class LayerRun:
+    """One run of a layer in the order of the forward pass."""
+    layer: int
+    cache: int                      # run whose cache or state it uses
+    enters: Optional[int] = None    # number of the loop pass it begins
 
 
 @dataclass(frozen=True)
@@ -156,14 +224,32 @@ class LayeredConfig:
     hidden_size: int
     layers: Tuple[LayerSpec, ...]
     rms_eps: float = 1e-6
+    norm_offset: float = 0.0        # added to the weights of stream norms
+    post_norms: bool = False        # sublayer outputs are normed as well
     embed_scale: float = 1.0
     max_position: int = 8192
+    learned_positions: bool = False     # a vector per position is embedded
+    loop: Optional[LoopSpec] = None
     vision_hidden: int = 0          # no multimodal tower
     weights_dir: str = ""           # checkpoint folder ("": random init)
 
     def __post_init__(self):
+        if self.loop is not None:
+            lp = self.loop
+            if not 0 <= lp.start < lp.stop <= len(self.layers) or \
+                    lp.times < 1:
+                raise ValueError(f"loop {lp.start}..{lp.stop} x {lp.times} "
+                                 f"over {len(self.layers)} layers")
         for i, layer in enumerate(self.layers):
-            m = layer.mixer
+            m, ff = layer.mixer, layer.ff
+            if isinstance(ff, ExpertsSpec) and not 0 < ff.top <= ff.experts:
+                raise ValueError(f"layer {i}: top {ff.top} of {ff.experts} "
+                                 "experts")
+            if isinstance(m, GroupedAttentionSpec):
+                if m.heads % m.kv_heads:
+                    raise ValueError(f"layer {i}: heads {m.heads} is not a "
+                                     f"multiple of kv_heads {m.kv_heads}")
+                continue
             if isinstance(m, ChannelDeltaSpec):
                 if m.heads % m.kv_heads:
                     raise ValueError(f"layer {i}: heads {m.heads} is not a "
@@ -196,20 +282,39 @@ class LayeredConfig:
         return len(self.layers)
 
     @property
+    def runs(self) -> Tuple[LayerRun, ...]:
+        """Layers in the order they run; every run has its own cache or
+        state, or shares that of the latest run of the layer it names."""
+        n = len(self.layers)
+        lp = self.loop or LoopSpec(n, n, 0)
+        order = [(i, None) for i in range(lp.start)]
+        for t in range(lp.times):
+            order += [(i, t if i == lp.start else None)
+                      for i in range(lp.start, lp.stop)]
+        order += [(i, None) for i in range(lp.stop, n)]
+        runs, latest = [], {}
+        for r, (i, enters) in enumerate(order):
+            latest[i] = r
+            source = getattr(self.layers[i].mixer, "kv_from", None)
+            runs.append(LayerRun(i, r if source is None else latest[source],
+                                 enters))
+        return tuple(runs)
+
+    @property
     def has_recurrent_state(self) -> bool:
         return any(isinstance(x.mixer, ChannelDeltaSpec)
                    for x in self.layers)
 
     def kv_bytes_per_token(self, dtype_bytes: int = 2) -> int:
-        return dtype_bytes * sum(
-            x.mixer.cache_width for x in self.layers
-            if isinstance(x.mixer, LatentAttentionSpec))
+        return dtype_bytes * sum(self.layers[r.layer].mixer.cache_width
+                                 for r in self.runs)
 
     def state_bytes_per_sequence(self, dtype_bytes: int = 2) -> int:
         total = 0
-        for x in self.layers:
-            if isinstance(x.mixer, ChannelDeltaSpec):
-                (h, k, v), (c, t) = x.mixer.state_shapes
+        for r in self.runs:
+            m = self.layers[r.layer].mixer
+            if isinstance(m, ChannelDeltaSpec):
+                (h, k, v), (c, t) = m.state_shapes
                 total += h * k * v * 4 + c * t * dtype_bytes
         return total
 
@@ -232,8 +337,9 @@ def _rururax(name, vocab, width, ff, heads, kv_heads, dim, q_rank, kv_rank,
                 scale=(dim + rot_dim) ** -0.5, rot=rot, window=window,
                 kv_from=own if kind == "s" else None)
             own = i if kind == "a" else own
-        layers.append(LayerSpec(mixer, ff))
+        layers.append(LayerSpec(mixer, GatedSpec(ff)))
     return LayeredConfig(name, "Rururax", vocab, width, tuple(layers),
+                         norm_offset=1.0, post_norms=True,
                          embed_scale=width ** 0.5, max_position=max_position)
 
 
@@ -245,3 +351,29 @@ TINY_RURURAX = _rururax("tiny-rururax", 768, 80, 112, heads=6, kv_heads=3,
                         dim=20, q_rank=40, kv_rank=48, window=24,
                         pattern="dads", rot_dim=12, lowrank=10,
                         attn_heads=5, conv=3, max_position=1024)
+
+
+def _sezazen(name, vocab, width, heads, kv_heads, dim, vdim, ff, experts, top,
+             expert_ff, shared_ff, pattern, loop=None, max_position=8192):
+    """A Sezazen stack: `pattern` is a string of d (dense feed-forward), e
+    (experts) and n (no feed-forward); loop = (start, stop, times)."""
+    mixer = GroupedAttentionSpec(heads, kv_heads, dim, vdim,
+                                 scale=dim ** -0.5, sink=0.0)
+    kinds = {"d": GatedSpec(ff, "silu"), "n": None,
+             "e": ExpertsSpec(experts, top, expert_ff, shared_ff)}
+    return LayeredConfig(name, "Sezazen", vocab, width,
+                         tuple(LayerSpec(mixer, kinds[k]) for k in pattern),
+                         learned_positions=True, max_position=max_position,
+                         loop=LoopSpec(*loop) if loop else None)
+
+
+# an 8B-class stack (about 6B of its weights run per token and pass), and a
+# small one for tests
+SEZAZEN_8B = _sezazen("sezazen-8b", 128256, 4096, heads=32, kv_heads=8,
+                      dim=128, vdim=128, ff=14336, experts=32, top=4,
+                      expert_ff=3584, shared_ff=7168,
+                      pattern="d" + "e" * 15, loop=(4, 12, 2))
+TINY_SEZAZEN = _sezazen("tiny-sezazen", 768, 72, heads=6, kv_heads=2, dim=20,
+                        vdim=28, ff=104, experts=6, top=2, expert_ff=24,
+                        shared_ff=40, pattern="edne", loop=(1, 3, 2),
+                        max_position=1024)

@@ -8,6 +8,11 @@ all rows as one product each; mixers split the rows by what suits them:
                    chunked kernels for the long portions after them
   LatentAttention  absorbed attention on the paged latents for the first
                    rows, expanded keys and values for the long portions
+  GroupedAttention both straight on the pages: parts of the context for the
+                   first rows, query tiles for the long portions
+
+The order of the forward is config.runs: a looped stretch of layers runs
+several times, every pass with caches of its own.
 
 The residual stream is 32-bit; activations are `dtype` (bf16, or float32 for
 exact runs). Mixers are independent of the design that lists them: a design
@@ -20,14 +25,15 @@ import numpy as np
 import torch
 
 from ..ops import layered as ops
-from .configs import (ChannelDeltaSpec, LatentAttentionSpec, LayeredConfig,
-                      RotarySpec)
-from . import rotary
+from ..ops.layered import linear
+from .configs import (ChannelDeltaSpec, GroupedAttentionSpec,
+                      LatentAttentionSpec, LayeredConfig, RotarySpec)
+from . import feed_forward, rotary
 
 # portions up to this many tokens run like decoded tokens
 SHORT = 8
 CHUNK = 64                  # tokens per chunk of the chunked recurrence
-QUERY_TILE = 128            # query rows per workgroup of latent_prefill
+QUERY_TILE = 128            # query rows per workgroup of the prefill kernels
 WORK_BYTES = 160 << 20      # its workspace: stays in the last-level cache
 
 
@@ -96,10 +102,6 @@ class LayeredBatch:
     max_ctx: int                    # longest context among the step rows
     long: List[Portion]
     logit_rows: Optional[torch.Tensor] = None   # None: every row
-
-
-def linear(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
-    return x @ w.t()
 
 
 class ChannelDelta:
@@ -205,8 +207,44 @@ class LatentAttention:
             lat = ops.gather_rows(cache, slots)
             kv = linear(lat[:, :s.kv_rank], self.w_ukv)
             ops.latent_prefill(q, kv, lat, batch.positions, batch.row_seq, n,
-                               batch.seq_meta, origin, ctx["tiles"],
+                               batch.seq_meta, origin,
+                               ctx["tiles", QUERY_TILE],
                                s.rot_dim, s.window, s.scale, out)
+        return linear(out, self.w_o)
+
+
+class GroupedAttention:
+    """Attention of grouped heads over paged keys and values."""
+
+    def __init__(self, spec: GroupedAttentionSpec, take: Callable,
+                 dtype: torch.dtype):
+        self.spec = spec
+        self.w_in = torch.cat([take(n) for n in "qkv"]).to(dtype)
+        self.w_o = take("o").to(dtype)
+
+    @property
+    def tile_rows(self) -> int:
+        """Queries of a portion per tile: the heads of a group share it."""
+        return max(1, QUERY_TILE * self.spec.kv_heads // self.spec.heads)
+
+    def __call__(self, h: torch.Tensor, batch: LayeredBatch, cache,
+                 ctx) -> torch.Tensor:
+        s, n = self.spec, batch.n_step_rows
+        T = h.shape[0]
+        proj = linear(h, self.w_in)
+        ops.store_heads(proj, s.heads * s.dim, batch.slot_mapping, cache,
+                        s.dim)
+        out = torch.empty((T, s.heads * s.vdim), dtype=h.dtype,
+                          device=h.device)
+        if n:
+            ops.grouped_decode(proj, cache, batch.positions, batch.row_seq,
+                               batch.block_tables, n, s.heads, s.dim,
+                               s.scale, s.sink, batch.max_ctx, out)
+        if n < T:
+            ops.grouped_prefill(proj, cache, batch.positions, batch.row_seq,
+                                batch.block_tables, n, batch.seq_meta,
+                                ctx["tiles", self.tile_rows], s.heads, s.dim,
+                                s.scale, s.sink, out)
         return linear(out, self.w_o)
 
 
@@ -221,41 +259,55 @@ class LayeredRunner:
         tables: Dict[RotarySpec, torch.Tensor] = {}
         self.embed = take("embed").to(dtype)
         self.lm_head = self.embed
-        self.mixers, self.norms, self.mlps, self.kv_layer = [], [], [], []
+        self.positions = take("pos").float() if config.learned_positions \
+            else None
+        self.runs = config.runs
+        self.loop_x = self.loop_x0 = self.loop_step = None
+        if config.loop:
+            w = take("loop.in").to(dtype)
+            self.loop_x = w[:, :config.hidden_size].contiguous()
+            self.loop_x0 = w[:, config.hidden_size:].contiguous()
+            self.loop_step = take("loop.step").float()
+        self.mixers, self.norms, self.mlps = [], [], []
         self.windows = set()
         for i, layer in enumerate(config.layers):
             m = layer.mixer
 
             def mix(name, i=i):
                 return take(f"l{i}.mix.{name}")
+
+            def mlp(name, i=i):
+                return take(f"l{i}.mlp.{name}")
             if isinstance(m, ChannelDeltaSpec):
                 self.mixers.append(ChannelDelta(m, mix, eps, dtype, device))
-                self.kv_layer.append(i)
+            elif isinstance(m, GroupedAttentionSpec):
+                self.mixers.append(GroupedAttention(m, mix, dtype))
             else:
                 if m.rot not in tables:
                     tables[m.rot] = rotary.table(m.rot, max_model_len, device)
                 self.mixers.append(LatentAttention(m, mix, eps, dtype,
                                                    tables[m.rot]))
-                self.kv_layer.append(i if m.kv_from is None else m.kv_from)
                 self.windows.add(m.window)
-            names = ("norm1", "norm1b") + (("norm2", "norm2b")
-                                           if layer.ff else ())
+            names = ("norm1",) + ("norm2",) * bool(layer.ff)
+            if config.post_norms:
+                names += tuple(n + "b" for n in names)
             self.norms.append({x: take(f"l{i}.{x}").float() for x in names})
-            self.mlps.append(None if not layer.ff else (
-                torch.cat([take(f"l{i}.mlp.gate"),
-                           take(f"l{i}.mlp.up")]).to(dtype),
-                take(f"l{i}.mlp.down").to(dtype)))
+            self.mlps.append(layer.ff and feed_forward.build(layer.ff, mlp,
+                                                             dtype))
         self.final_norm = take("final.norm").float()
+        # query tiles the prefill kernels take, by queries per tile
+        self.tile_rows = {m.tile_rows for m in self.mixers
+                          if isinstance(m, GroupedAttention)}
+        if self.windows:
+            self.tile_rows.add(QUERY_TILE)
 
     def weight_bytes(self) -> int:
         seen, total = set(), 0
-        for obj in [self] + self.mixers:
+        for obj in [self] + self.mixers + [m for m in self.mlps if m]:
             for t in vars(obj).values():
                 if isinstance(t, torch.Tensor) and t.data_ptr() not in seen:
                     seen.add(t.data_ptr())
                     total += t.numel() * t.element_size()
-        for pair in self.mlps:
-            total += sum(t.numel() * t.element_size() for t in pair or ())
         return total
 
     # ------------------------------------------------------------------
@@ -275,41 +327,54 @@ class LayeredRunner:
         return (torch.from_numpy(np.concatenate(slots)).to(self.device),
                 torch.from_numpy(origin).to(self.device))
 
+    def _shared_inputs(self, batch: LayeredBatch, block_size: int) -> dict:
+        """What layers of equal sizes share about the long portions."""
+        ctx = {}
+        if not batch.long:
+            return ctx
+        for n in self.tile_rows:
+            ctx["tiles", n] = torch.tensor(
+                [(p.seq, r) for p in batch.long for r in range(0, p.n, n)],
+                dtype=torch.int32).to(self.device)
+        for w in self.windows:
+            ctx["keys", w] = self._context(batch, w, block_size)
+        for n in {m.per_group for m in self.mixers
+                  if isinstance(m, ChannelDelta) and m.work}:
+            ctx["chunks", n] = chunk_groups(batch.long, n, self.device)
+        return ctx
+
     def forward(self, batch: LayeredBatch, pool,
                 embeddings_out: bool = False,
                 layers_out: Optional[list] = None) -> torch.Tensor:
         """-> logits of `logit_rows` (or the normed stream of every row).
-        layers_out collects copies of the stream after every layer."""
-        c = self.cfg
-        ctx = {}            # what layers of equal sizes share
-        if batch.long:
-            if self.windows:
-                ctx["tiles"] = torch.tensor(
-                    [(p.seq, r) for p in batch.long
-                     for r in range(0, p.n, QUERY_TILE)],
-                    dtype=torch.int32).to(self.device)
-            for w in self.windows:
-                ctx["keys", w] = self._context(batch, w, pool.block_size)
-            for n in {m.per_group for m in self.mixers
-                      if isinstance(m, ChannelDelta) and m.work}:
-                ctx["chunks", n] = chunk_groups(batch.long, n, self.device)
-        pre = [n["norm1"] for n in self.norms] + [self.final_norm]
+        layers_out collects copies of the stream after every layer run."""
+        c, runs = self.cfg, self.runs
+        ctx = self._shared_inputs(batch, pool.block_size)
+        # the norm ahead of every run; a run that enters a loop pass takes
+        # the stream itself (None)
+        pre = [None if r.enters is not None else self.norms[r.layer]["norm1"]
+               for r in runs] + [self.final_norm]
 
-        def norm(y, post, following):
-            return ops.stream_norm(x, y, post, following, 1.0, c.rms_eps,
-                                   self.dtype)
+        def update(y, rows, post, following):
+            return ops.stream_norm(x, y, post, following, c.norm_offset,
+                                   c.rms_eps, self.dtype, rows)
         x, h = ops.embed_norm(batch.input_ids, self.embed, c.embed_scale,
-                              pre[0], 1.0, c.rms_eps)
-        for i, mixer in enumerate(self.mixers):
-            norms = self.norms[i]
-            y = mixer(h, batch, pool.layers[self.kv_layer[i]], ctx)
-            if self.mlps[i] is not None:
-                h = norm(y, norms["norm1b"], norms["norm2"])
-                gate_up, down = self.mlps[i]
-                y = linear(ops.gelu_mul(linear(h, gate_up)), down)
-                h = norm(y, norms["norm2b"], pre[i + 1])
-            else:
-                h = norm(y, norms["norm1b"], pre[i + 1])
+                              pre[0], c.norm_offset, c.rms_eps,
+                              self.positions, batch.positions)
+        if c.loop:      # the embedding output's share is the same every pass
+            x0 = ops.linear32(h if pre[0] is None else x.to(self.dtype),
+                              self.loop_x0)
+        for i, run in enumerate(runs):
+            norms, mlp = self.norms[run.layer], self.mlps[run.layer]
+            if run.enters is not None:
+                h = ops.loop_norm(x, ops.linear32(h, self.loop_x), x0,
+                                  self.loop_step[run.enters], norms["norm1"],
+                                  c.norm_offset, c.rms_eps, self.dtype)
+            y = self.mixers[run.layer](h, batch, pool.layers[run.cache], ctx)
+            h = update(y, None, norms.get("norm1b"),
+                       norms["norm2"] if mlp else pre[i + 1])
+            if mlp:
+                h = update(*mlp(h), norms.get("norm2b"), pre[i + 1])
             if layers_out is not None:
                 layers_out.append(x.clone())
         if embeddings_out:

@@ -10,7 +10,7 @@ from typing import Union
 
 import torch
 
-from . import configs, rururax
+from . import checkpoint, configs, rururax, sezazen
 from .configs import LayeredConfig, ModelConfig
 
 AnyConfig = Union[ModelConfig, LayeredConfig]
@@ -18,13 +18,12 @@ AnyConfig = Union[ModelConfig, LayeredConfig]
 MODELS = {c.name: c for c in (
     configs.LLAMA_3_8B, configs.QWEN3_32B, configs.LLAVA_1_5_7B_TEXT,
     configs.TINY_LLAMA, configs.TINY_QWEN, configs.TINY_LLAVA,
-    configs.RURURAX_8B, configs.TINY_RURURAX)}
+    configs.RURURAX_8B, configs.TINY_RURURAX, configs.SEZAZEN_8B,
+    configs.TINY_SEZAZEN)}
 
-# config.json "architecture" -> reader of the folder's configuration
-READERS = {rururax.ARCHITECTURE: rururax.read_config}
-
-# LayeredConfig.architecture -> supplier of named weights for the runner
-WEIGHTS = {rururax.ARCHITECTURE: rururax.weights}
+# config.json "architecture" (LayeredConfig.architecture) -> module with the
+# design's read_config, tensor_shapes and random_tensor
+DESIGNS = {d.ARCHITECTURE: d for d in (rururax, sezazen)}
 
 
 def resolve(model: str) -> AnyConfig:
@@ -38,9 +37,9 @@ def resolve(model: str) -> AnyConfig:
     with open(path) as f:
         raw = json.load(f)
     arch = raw.get("architecture")
-    if arch not in READERS:
+    if arch not in DESIGNS:
         raise ValueError(f"{path}: unknown architecture {arch!r}")
-    return READERS[arch](raw, model)
+    return DESIGNS[arch].read_config(raw, model)
 
 
 def build_runner(config: AnyConfig, device: torch.device,
@@ -50,6 +49,9 @@ def build_runner(config: AnyConfig, device: torch.device,
         from .llama import LlamaRunner
         return LlamaRunner(config, device, dtype, seed=seed)
     from .layered import LayeredRunner
-    return LayeredRunner(config, WEIGHTS[config.architecture](
-        config, device, dtype, seed), device, dtype,
-        max_model_len=max_model_len)
+    design = DESIGNS[config.architecture]
+    take = checkpoint.weights(config.weights_dir,
+                              design.tensor_shapes(config),
+                              design.random_tensor, device, seed)
+    return LayeredRunner(config, take, device, dtype,
+                         max_model_len=max_model_len)

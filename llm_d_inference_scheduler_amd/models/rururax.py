@@ -1,4 +1,4 @@
-"""Rururax: configuration reader and weights (files or random init).
+"""Rururax: configuration reader, tensor names and random init.
 
 A stack of gated-delta-rule layers with per-channel decay and latent
 attention layers (some of which attend to an earlier layer's cached
@@ -12,12 +12,9 @@ from typing import Any, Callable, Dict
 
 import torch
 
-from ..utils.logging import get_logger
 from .checkpoint import read_safetensors
-from .configs import (ChannelDeltaSpec, LatentAttentionSpec, LayeredConfig,
-                      LayerSpec, RotarySpec)
-
-log = get_logger("models.rururax")
+from .configs import (ChannelDeltaSpec, GatedSpec, LatentAttentionSpec,
+                      LayeredConfig, LayerSpec, RotarySpec)
 
 ARCHITECTURE = "Rururax"
 
@@ -59,12 +56,12 @@ def read_config(raw: Dict[str, Any], folder: str) -> LayeredConfig:
         mlp = entry.get("mlp")
         if mlp and mlp["kind"] != "dense":
             raise ValueError(f"layer {i}: unknown mlp {mlp['kind']!r}")
-        layers.append(LayerSpec(mixer, mlp["ff"] if mlp else None))
+        layers.append(LayerSpec(mixer, GatedSpec(mlp["ff"]) if mlp else None))
     return LayeredConfig(
         name=os.path.basename(os.path.normpath(folder)) or "rururax",
         architecture=ARCHITECTURE, vocab_size=raw["vocab"],
         hidden_size=raw["width"], layers=tuple(layers),
-        rms_eps=float(raw["norm"]["eps"]),
+        rms_eps=float(raw["norm"]["eps"]), norm_offset=1.0, post_norms=True,
         embed_scale=float(raw["embedding"]["scale"]), weights_dir=folder)
 
 
@@ -99,8 +96,8 @@ def tensor_shapes(c: LayeredConfig) -> Dict[str, tuple]:
         for k, shape in mix.items():
             out[p + "mix." + k] = shape
         if layer.ff:
-            out[p + "mlp.gate"] = out[p + "mlp.up"] = (layer.ff, w)
-            out[p + "mlp.down"] = (w, layer.ff)
+            out[p + "mlp.gate"] = out[p + "mlp.up"] = (layer.ff.ff, w)
+            out[p + "mlp.down"] = (w, layer.ff.ff)
     return out
 
 
@@ -117,37 +114,3 @@ def random_tensor(name: str, shape: tuple, fill: Callable) -> torch.Tensor:
     if leaf == "mix.dt_bias":
         return fill(shape, 1.0).sub_(3.0)
     return fill(shape, 1.0 / math.sqrt(shape[-1]))
-
-
-def weights(c: LayeredConfig, device: torch.device, dtype: torch.dtype,
-            seed: int) -> Callable[[str], torch.Tensor]:
-    """-> take(name): the tensor in its stored precision on `device`."""
-    shapes = tensor_shapes(c)
-    if c.weights_dir:
-        files = read_safetensors(os.path.join(c.weights_dir,
-                                              "model.safetensors"))
-        missing = sorted(set(shapes) - set(files))
-        if missing:
-            raise ValueError(f"{c.weights_dir}: missing tensors {missing}")
-        if len(files) > len(shapes):
-            log.warning("unused tensors", names=sorted(set(files)
-                                                       - set(shapes)))
-
-        def take(name):
-            t = files[name]
-            if tuple(t.shape) != shapes[name]:
-                raise ValueError(f"{name}: shape {tuple(t.shape)}, expected "
-                                 f"{shapes[name]}")
-            return t.to(device)
-        return take
-    # drawn on the device itself: a checkpoint-sized CPU init would dominate
-    # start-up. One seed gives every rank the same weights.
-    gen = torch.Generator(device=device).manual_seed(seed)
-
-    def take(name):
-        def fill(shape, std):
-            return torch.empty(shape, dtype=torch.float32,
-                               device=device).normal_(0.0, std,
-                                                      generator=gen)
-        return random_tensor(name, shapes[name], fill).to(torch.bfloat16)
-    return take

@@ -23,21 +23,61 @@ def _impl(t: torch.Tensor):
     return hip_layered() if t.is_cuda else ref
 
 
-def embed_norm(ids, table, scale, wn, offset, eps):
-    """-> (stream x = table[ids] * scale in 32-bit, its norm)."""
-    return _impl(table).embed_norm(ids, table, scale, wn, offset, eps)
+# activation codes of the kernels
+ACTS = {"gelu_tanh": 0, "silu": 1, "relu_squared": 2}
 
 
-def stream_norm(x, y, wb, wn, offset, eps, dtype):
-    """x += rms_norm(y) * (wb + offset), in place (skipped without y);
-    -> rms_norm(x) * (wn + offset) as dtype."""
+def linear(x, w):
+    return x @ w.t()
+
+
+def linear32(x, w):
+    """x @ w' with a 32-bit result."""
+    if x.is_cuda and x.dtype != torch.float32:
+        return torch.mm(x, w.t(), out_dtype=torch.float32)
+    return x.float() @ w.float().t()
+
+
+def embed_norm(ids, table, scale, wn, offset, eps, pos=None, positions=None):
+    """-> (stream x = table[ids] * scale (+ pos[positions]) in 32-bit, its
+    norm; without wn x itself in the table's type)."""
+    return _impl(table).embed_norm(ids, table, scale, wn, offset, eps, pos,
+                                   positions)
+
+
+def stream_norm(x, y, wb, wn, offset, eps, dtype, rows=None):
+    """In place: x += rms_norm(y) * (wb + offset), without wb x += y, without
+    y nothing; with rows [T * n, width] also each token's n rows.
+    -> rms_norm(x) * (wn + offset) as dtype; without wn x as dtype."""
     return _impl(x).stream_norm(x, y, wb, wn, offset, eps,
-                                dtype == torch.float32)
+                                dtype == torch.float32, rows)
 
 
-def gelu_mul(gate_up):
-    """gelu_tanh(gate) * up on packed rows."""
-    return _impl(gate_up).gelu_mul(gate_up)
+def loop_norm(x, a, b, v, wn, offset, eps, dtype):
+    """In place: x = a + b + v (a vector); -> its norm as in stream_norm."""
+    return _impl(x).loop_norm(x, a, b, v, wn, offset, eps,
+                              dtype == torch.float32)
+
+
+def gated_act(gate_up, act):
+    """act(gate) * up on packed rows."""
+    return _impl(gate_up).gated_act(gate_up, ACTS[act])
+
+
+def activate(x, act):
+    return _impl(x).activate(x, ACTS[act])
+
+
+def route(h, w, top):
+    """-> (experts [T, top] int32 with the largest scores sigmoid(h w'),
+    largest first, and these scores), scores in 32-bit."""
+    return _impl(h).route(h, w, top)
+
+
+def experts(h, ids, weights, up, down, act, plain=False):
+    """down[e] act(up[e] (weight h)) of every token's experts e, rows
+    [T * top, width] in the order of ids."""
+    return _impl(h).experts(h, ids, weights, up, down, ACTS[act], plain)
 
 
 def delta_prep(proj, taps, conv_state, row_seq, seq_meta, multi_row, kv_heads,
@@ -109,3 +149,28 @@ def latent_prefill(q, kv, lat, positions, row_seq, base, seq_meta, ctx, tiles,
     """Attention of the rows from `base` on over expanded keys and values."""
     _impl(q).latent_prefill(q, kv, lat, positions, row_seq, base, seq_meta,
                             ctx, tiles, rot, window or 0, scale, out, plain)
+
+
+def store_heads(proj, col, slots, cache, dim):
+    """Keys of all heads, then values of all heads, from column `col` on ->
+    the cache pages [blocks, heads, tokens, key | value]."""
+    _impl(proj).store_heads(proj, col, slots, cache, dim)
+
+
+def grouped_decode(proj, cache, positions, row_seq, block_tables, n, heads,
+                   dim, scale, sink, max_ctx, out, plain=False):
+    """Attention of the first n rows (queries lead the rows of proj) over the
+    paged keys and values; sink: score of a key without a value, or None."""
+    _impl(proj).grouped_decode(proj, cache, positions, row_seq, block_tables,
+                               n, heads, dim, scale, sink, max_ctx, out,
+                               plain)
+
+
+def grouped_prefill(proj, cache, positions, row_seq, block_tables, base,
+                    seq_meta, tiles, heads, dim, scale, sink, out,
+                    plain=False):
+    """The same for the rows from `base` on; tiles [n, 2] = (sequence, first
+    row of its portion)."""
+    _impl(proj).grouped_prefill(proj, cache, positions, row_seq,
+                                block_tables, base, seq_meta, tiles, heads,
+                                dim, scale, sink, out, plain)

@@ -9,22 +9,60 @@ def _rms(x, w, offset, eps):
         (w + offset)
 
 
-def embed_norm(ids, table, scale, wn, offset, eps):
-    x = table[ids].float() * scale
-    return x, _rms(x, wn, offset, eps).to(table.dtype)
-
-
-def stream_norm(x, y, wb, wn, offset, eps, f32):
-    if y is not None:
-        x += _rms(y, wb, offset, eps)
-    return _rms(x, wn, offset, eps).to(
+def _out(x, wn, offset, eps, f32):
+    return (x if wn is None else _rms(x, wn, offset, eps)).to(
         torch.float32 if f32 else torch.bfloat16)
 
 
-def gelu_mul(gate_up):
+def embed_norm(ids, table, scale, wn, offset, eps, pos, positions):
+    x = table[ids].float() * scale
+    if pos is not None:
+        x += pos[positions.long()]
+    return x, _out(x, wn, offset, eps, table.dtype == torch.float32)
+
+
+def stream_norm(x, y, wb, wn, offset, eps, f32, rows):
+    if y is not None:
+        x += y if wb is None else _rms(y, wb, offset, eps)
+    if rows is not None:
+        x += rows.float().view(x.shape[0], -1, x.shape[1]).sum(1)
+    return _out(x, wn, offset, eps, f32)
+
+
+def loop_norm(x, a, b, v, wn, offset, eps, f32):
+    x.copy_(a + b + v)
+    return _out(x, wn, offset, eps, f32)
+
+
+def _act(z, act):
+    if act == 0:
+        return torch.nn.functional.gelu(z, approximate="tanh")
+    return torch.nn.functional.silu(z) if act == 1 else z.clamp(min=0) ** 2
+
+
+def gated_act(gate_up, act):
     g, u = gate_up.float().chunk(2, -1)
-    return (torch.nn.functional.gelu(g, approximate="tanh") * u).to(
-        gate_up.dtype)
+    return (_act(g, act) * u).to(gate_up.dtype)
+
+
+def activate(x, act):
+    return _act(x.float(), act).to(x.dtype)
+
+
+def route(h, w, top):
+    z, ids = (h.float() @ w.float().t()).topk(top)
+    return ids.int(), torch.sigmoid(z)
+
+
+def experts(h, ids, weights, up, down, act, plain):
+    top = ids.shape[1]
+    out = torch.empty((ids.numel(), h.shape[1]), dtype=h.dtype)
+    for e in range(up.shape[0]):
+        pairs = (ids.flatten() == e).nonzero().flatten()
+        z = h[pairs // top].float() @ up[e].float().t()
+        hid = _act(z * weights.flatten()[pairs, None], act).to(h.dtype)
+        out[pairs] = (hid.float() @ down[e].float().t()).to(h.dtype)
+    return out
 
 
 def delta_prep(proj, taps, conv_state, row_seq, seq_meta, multi_row, kv_heads,
@@ -142,3 +180,38 @@ def latent_prefill(q, kv, lat, positions, row_seq, base, seq_meta, ctx, tiles,
             q[i, :, D:].float() @ kr[a:b].T
         o = torch.einsum("ht,thv->hv", torch.softmax(s * scale, -1), v[a:b])
         out[i] = o.flatten().to(out.dtype)
+
+
+def store_heads(proj, col, slots, cache, dim):
+    G, bs, W = cache.shape[1:]
+    rows, split = proj.shape[0], col + G * dim
+    new = torch.cat([proj[:, col:split].view(rows, G, dim),
+                     proj[:, split:].view(rows, G, W - dim)], -1)
+    cache[slots // bs, :, slots % bs] = new
+
+
+def _grouped(proj, cache, positions, row_seq, block_tables, lo, hi, heads,
+             dim, scale, sink, out):
+    G, bs = cache.shape[1:3]
+    for i in range(lo, hi):
+        t = torch.arange(int(positions[i]) + 1)
+        blocks = block_tables[int(row_seq[i])].long()[t // bs]
+        kv = cache[blocks, :, t % bs].float().transpose(0, 1)   # [G, t, W]
+        q = proj[i, :heads * dim].float().view(G, heads // G, dim)
+        s = q @ kv[..., :dim].transpose(1, 2) * scale
+        if sink is not None:
+            s = torch.cat([s, torch.full_like(s[..., :1], sink)], -1)
+        p = torch.softmax(s, -1)[..., :len(t)]
+        out[i] = (p @ kv[..., dim:]).flatten().to(out.dtype)
+
+
+def grouped_decode(proj, cache, positions, row_seq, block_tables, n, heads,
+                   dim, scale, sink, max_ctx, out, plain):
+    _grouped(proj, cache, positions, row_seq, block_tables, 0, n, heads, dim,
+             scale, sink, out)
+
+
+def grouped_prefill(proj, cache, positions, row_seq, block_tables, base,
+                    seq_meta, tiles, heads, dim, scale, sink, out, plain):
+    _grouped(proj, cache, positions, row_seq, block_tables, base,
+             proj.shape[0], heads, dim, scale, sink, out)

@@ -8,7 +8,8 @@ files live inside the package and travel with the repo snapshot:
     extension, hipcc --offload-arch=gfx950): prefix hash/match, paged KV,
     fused norm/rope/act, GQA decode attention.
   * llm_d_inference_scheduler_amd._hip_layered  — gfx950 HIP kernels of the
-    layer-listed designs (delta rule, latent attention, 32-bit stream).
+    layer-listed designs (delta rule, latent and grouped attention,
+    experts, 32-bit stream).
 
 LDS_AMD_ONLY=name,... builds only the named modules (e.g. _hip_layered).
 """
@@ -60,9 +61,11 @@ hip_layered = cpp_extension.CUDAExtension(
         "csrc/hip/layered/residual_norm.hip",
         "csrc/hip/layered/delta_rule.hip",
         "csrc/hip/layered/delta_chunk.hip",
-        "csrc/hip/layered/latent_attention.hip",
-        "csrc/hip/layered/latent_decode.hip",
-        "csrc/hip/layered/latent_prefill.hip",
+        "csrc/hip/layered/attention.hip",
+        "csrc/hip/layered/paged_decode.hip",
+        "csrc/hip/layered/context_prefill.hip",
+        "csrc/hip/layered/experts.hip",
+        "csrc/hip/layered/ops_grouped.hip",
     ],
     extra_compile_args=HIP_ARGS,
 )
