@@ -1078,7 +1078,7 @@ class EngineWorker:
                           torch.ones_like(temps))
         y = logits.float() * inv.unsqueeze(1)
         u = torch.rand_like(y).clamp_min(1e-20)
-        gumbel = -torch.log(-torch.log(u).clamp_min(1e-20))
+        gumbel = -torch.log((-torch.log(u)).clamp_min(1e-20))
         y = y + gumbel * hot.unsqueeze(1)
         return y.argmax(dim=-1)
 

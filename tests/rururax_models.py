@@ -1,11 +1,12 @@
 """Small Rururax models for the tests: configurations in the checkpoint's own
 keys, random weights, and a folder writer."""
 import copy
-import json
 import math
-import os
 
 import torch
+
+import model_files
+from model_files import tokens  # noqa: F401
 
 # sizes no kernel has a vector form for: odd groups, unequal dims, two
 # windows, a layer without feed-forward, plain rotary
@@ -119,30 +120,10 @@ def random_weights(cfg, seed=0):
     return out
 
 
-def write_safetensors(path, tensors):
-    names = {torch.bfloat16: "BF16", torch.float32: "F32",
-             torch.int32: "I32"}
-    header, blobs, at = {}, [], 0
-    for k, t in tensors.items():
-        raw = t.contiguous().view(torch.uint8).numpy().tobytes() \
-            if t.dim() else b""
-        header[k] = {"dtype": names[t.dtype], "shape": list(t.shape),
-                     "data_offsets": [at, at + len(raw)]}
-        blobs.append(raw)
-        at += len(raw)
-    head = json.dumps(header).encode()
-    with open(path, "wb") as f:
-        f.write(len(head).to_bytes(8, "little") + head + b"".join(blobs))
-
-
 def write_model(folder, cfg, weights=None, seed=0):
     """-> (folder path, weights)."""
-    os.makedirs(folder, exist_ok=True)
-    weights = random_weights(cfg, seed) if weights is None else weights
-    with open(os.path.join(folder, "config.json"), "w") as f:
-        json.dump(cfg, f)
-    write_safetensors(os.path.join(folder, "model.safetensors"), weights)
-    return str(folder), weights
+    return model_files.write_model(
+        folder, cfg, random_weights(cfg, seed) if weights is None else weights)
 
 
 def variant(cfg, **changes):
@@ -154,8 +135,3 @@ def variant(cfg, **changes):
             if k in layer["mixer"]:
                 layer["mixer"][k] = v
     return cfg
-
-
-def tokens(cfg, n, seed=0):
-    g = torch.Generator().manual_seed(1000 + seed)
-    return torch.randint(0, cfg["vocab"], (n,), generator=g).tolist()
