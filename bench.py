@@ -36,8 +36,11 @@ def parse_args():
                    choices=["mono", "pd", "fc", "epd", "layers"],
                    help="mono=prefix-aware DP decode; pd=P/D disagg; "
                         "fc=flow control at overload; epd=E/P/D multimodal; "
-                        "layers=prefill and decode of Rururax layers beside "
-                        "Llama layers of equal size (one GPU)")
+                        "layers=prefill and decode of a layer-listed "
+                        "design beside Llama layers of equal size (one GPU)")
+    p.add_argument("--layer-design", default="rururax",
+                   choices=["rururax", "sezazen"],
+                   help="design of --mode layers")
     p.add_argument("--layer-sizes", default="2b,8b,32b",
                    help="sizes of --mode layers, comma-separated")
     p.add_argument("--model", default="llama-3-8b",
@@ -512,19 +515,20 @@ def layers_main(args):
                              device="cpu")
     sizes = args.layer_sizes.split(",") if gpu else ["tiny"]
     steps = min(args.steps, 64)
-    rows = layer_bench.run(sizes, steps=steps, **kw)
-    last = [v for k, v in rows.items() if "/rururax/" in k][-1]
+    design = args.layer_design
+    rows = layer_bench.run(sizes, design, steps=steps, **kw)
+    last = [v for k, v in rows.items() if f"/{design}/" in k][-1]
     print(json.dumps({
-        "metric": "Rururax layers: prefill and decode tok/s beside Llama "
-                  "layers of equal size",
+        "metric": f"{design.capitalize()} layers: prefill and decode tok/s "
+                  "beside Llama layers of equal size",
         "value": last["decode_tok_s"], "unit": "tok/s", "n_gpus": 1,
         "steps": steps, "warmup": 8,
         "ms_per_step": last["decode_ms_per_step"],
         "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
         "dtype": "bf16" if gpu else "fp32",
         "data": "synthetic prompts, random-init weights",
-        "config": {"model": "rururax layers vs llama layers",
-                   "layers": layer_bench.PATTERN, "parallelism": "dp1",
+        "config": {"model": f"{design} layers vs llama layers",
+                   "layer_runs": layer_bench.RUNS, "parallelism": "dp1",
                    "results": rows}}), flush=True)
 
 

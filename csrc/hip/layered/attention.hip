@@ -1,6 +1,7 @@
-// latent_attention.hip — attention over a low-rank latent shared by all heads.
+// attention.hip — cache rows of latent attention and of grouped heads, and
+// plain attention over either.
 //
-// Cached per token: [latent (kv_rank, normed) | rotated key part (rot_dim)],
+// Latent attention caches per token: [latent (kv_rank, normed) | rotated key part (rot_dim)],
 // pages [n_blocks, block_size, kv_rank + rot_dim]. Rows that come alone (or
 // in short portions) attend to the pages directly, with the key projection
 // absorbed into the query; long portions expand keys and values first

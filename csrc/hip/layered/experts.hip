@@ -1,5 +1,5 @@
-// experts.hip — feed-forward experts: the router, tokens sorted by expert, and
-// the experts' products over the sorted (token, expert) pairs.
+// experts.hip — feed-forward experts: the router, (token, expert) pairs sorted
+// by expert, and the experts' products over them.
 //
 // A pair's inner row is act(weight * up[e] h): the weight scales the expert's
 // input, and since the product is linear it is applied to the 32-bit sums.
@@ -323,7 +323,8 @@ constexpr int TG = 8;                // tiles of pairs that run side by side
 
 template <bool UP>
 __global__ __launch_bounds__(256, 2) void expert_tiles_kernel(const Pairs p) {
-  __shared__ __align__(16) short lds[2][2][BT * BK];  // [buffer][weights, pairs]
+  // [buffer][weights, pairs]
+  __shared__ __align__(16) short lds[2][2][BT * BK];
   const int N = p.N, K = p.K;
   // Workgroups go round the 8 XCDs in turn: each XCD gets a contiguous share
   // of the work, in which TG tiles of pairs walk the channels together.

@@ -1,32 +1,56 @@
 """Prefill and decode throughput of a layer-listed design beside Llama at
-equal layer size (`bench.py --mode layers`): random weights, a stack of a few
-layers, the engine's own steps."""
+equal layer size (`bench.py --mode layers`): random weights, a stack of eight
+layer runs, the engine's own steps."""
 import sys
 import time
 
 import torch
 
-from ..models.configs import ModelConfig, _rururax
+from ..models.configs import LayeredConfig, ModelConfig, _rururax, _sezazen
 from .worker import EngineRequest, EngineWorker
 
-PATTERN = "ddda" + "ddds"
 VOCAB = 32768
-# name -> width, ff, heads, query rank, latent rank
-SIZES = {"tiny": (64, 128, 2, 32, 32),      # CPU smoke of the harness
-         "2b": (2048, 8192, 16, 768, 512),
-         "8b": (4096, 14336, 32, 1536, 512),
-         "32b": (5120, 25600, 64, 1536, 512)}
+# name -> width, ff, heads
+SIZES = {"tiny": (64, 128, 2),              # CPU smoke of the harness
+         "2b": (2048, 8192, 16),
+         "8b": (4096, 14336, 32),
+         "32b": (5120, 25600, 64)}
+RUNS = 8
+# query and latent rank
+RANKS = {"tiny": (32, 32), "2b": (768, 512), "8b": (1536, 512),
+         "32b": (1536, 512)}
+# experts, top, inner size of an expert and of the shared one: a token uses as
+# many feed-forward weights as in Llama's gated MLP
+EXPERTS = {"tiny": (8, 4, 32, 64), "2b": (32, 4, 2048, 4096),
+           "8b": (32, 4, 3584, 7168), "32b": (32, 4, 6400, 12800)}
 
 
-def configs(size: str, pattern: str = PATTERN):
-    width, ff, heads, q_rank, kv_rank = SIZES[size]
-    return {
-        "rururax": _rururax(f"rururax-{size}-layers", VOCAB, width, ff,
-                            heads=heads, kv_heads=heads, dim=128,
-                            q_rank=q_rank, kv_rank=kv_rank, window=1024,
-                            pattern=pattern),
-        "llama": ModelConfig(f"llama-{size}-layers", VOCAB, width, ff,
-                             len(pattern), heads, min(8, heads), 128)}
+def _rururax_stack(size: str) -> LayeredConfig:
+    width, ff, heads = SIZES[size]
+    q_rank, kv_rank = RANKS[size]
+    return _rururax(f"rururax-{size}-layers", VOCAB, width, ff, heads=heads,
+                    kv_heads=heads, dim=128, q_rank=q_rank, kv_rank=kv_rank,
+                    window=1024, pattern="dddaddds")
+
+
+def _sezazen_stack(size: str) -> LayeredConfig:
+    """Six layers, two of which run twice."""
+    width, ff, heads = SIZES[size]
+    experts, top, expert_ff, shared_ff = EXPERTS[size]
+    return _sezazen(f"sezazen-{size}-layers", VOCAB, width, heads=heads,
+                    kv_heads=min(8, heads), dim=128, vdim=128, ff=ff,
+                    experts=experts, top=top, expert_ff=expert_ff,
+                    shared_ff=shared_ff, pattern="deeeee", loop=(1, 3, 2))
+
+
+DESIGNS = {"rururax": _rururax_stack, "sezazen": _sezazen_stack}
+
+
+def configs(size: str, design: str):
+    width, ff, heads = SIZES[size]
+    return {design: DESIGNS[design](size),
+            "llama": ModelConfig(f"llama-{size}-layers", VOCAB, width, ff,
+                                 RUNS, heads, min(8, heads), 128)}
 
 
 def measure(cfg, prompts: int, prompt_len: int, batch: int, steps: int,
@@ -78,19 +102,16 @@ def measure(cfg, prompts: int, prompt_len: int, batch: int, steps: int,
             "decode_ms_per_step": round(dec * 1e3 / steps, 3)}
 
 
-def run(sizes, models=("rururax", "llama"), prompts: int = 8,
+def run(sizes, design: str = "rururax", prompts: int = 8,
         prompt_len: int = 1024, batches=(32, 256), steps: int = 32,
-        pattern: str = PATTERN, device: str = "cuda:0") -> dict:
+        device: str = "cuda:0") -> dict:
     out = {}
     for size in sizes:
-        cfgs = configs(size, pattern)
         for b in batches:
-            for name in models:     # both sides in turn
-                out[f"{size}/{name}/batch{b}"] = measure(
-                    cfgs[name], prompts, prompt_len, b, steps, device)
+            for name, cfg in configs(size, design).items():  # both in turn
+                key = f"{size}/{name}/batch{b}"
+                out[key] = measure(cfg, prompts, prompt_len, b, steps, device)
                 if device != "cpu":
                     torch.cuda.empty_cache()
-                print(f"{size}/{name}/batch{b}",
-                      out[f"{size}/{name}/batch{b}"], file=sys.stderr,
-                      flush=True)
+                print(key, out[key], file=sys.stderr, flush=True)
     return out

@@ -50,8 +50,9 @@ def activate(x, act):
 
 
 def route(h, w, top):
-    z, ids = (h.float() @ w.float().t()).topk(top)
-    return ids.int(), torch.sigmoid(z)
+    z, ids = (h.float() @ w.float().t()).sort(dim=-1, descending=True,
+                                              stable=True)
+    return ids[:, :top].int(), torch.sigmoid(z[:, :top])
 
 
 def experts(h, ids, weights, up, down, act, plain):
@@ -184,9 +185,9 @@ def latent_prefill(q, kv, lat, positions, row_seq, base, seq_meta, ctx, tiles,
 
 def store_heads(proj, col, slots, cache, dim):
     G, bs, W = cache.shape[1:]
-    rows, split = proj.shape[0], col + G * dim
-    new = torch.cat([proj[:, col:split].view(rows, G, dim),
-                     proj[:, split:].view(rows, G, W - dim)], -1)
+    k, v = proj[:, col:col + G * W].split([G * dim, G * (W - dim)], 1)
+    new = torch.cat([k.unflatten(1, (G, dim)),
+                     v.unflatten(1, (G, W - dim))], -1)
     cache[slots // bs, :, slots % bs] = new
 
 

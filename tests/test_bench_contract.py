@@ -6,6 +6,8 @@ import os
 import subprocess
 import sys
 
+import pytest
+
 REPO = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 
 REQUIRED = ["metric", "value", "unit", "n_gpus", "steps", "warmup",
@@ -57,18 +59,19 @@ def test_bench_multirank_contract():
     assert r["value"] > 0
 
 
-def test_bench_layers_mode():
+@pytest.mark.parametrize("design", ["rururax", "sezazen"])
+def test_bench_layers_mode(design):
     """`--mode layers` prints one JSON line with both designs' numbers."""
     out = subprocess.run(
         [sys.executable, "bench.py", "--mode", "layers", "--device", "cpu",
-         "--steps", "2"],
+         "--layer-design", design, "--steps", "2"],
         cwd=REPO, capture_output=True, text=True, timeout=300)
     assert out.returncode == 0, out.stderr[-2000:]
     lines = [l for l in out.stdout.splitlines() if l.startswith("{")]
     assert len(lines) == 1
     r = json.loads(lines[0])
     assert not [k for k in REQUIRED if k not in r]
-    assert set(r["config"]["results"]) == {"tiny/rururax/batch2",
+    assert set(r["config"]["results"]) == {f"tiny/{design}/batch2",
                                            "tiny/llama/batch2"}
     for row in r["config"]["results"].values():
         assert row["prefill_tok_s"] > 0 and row["decode_tok_s"] > 0

@@ -207,7 +207,7 @@ class TestFarKeys:
         weights = M.random_weights(M.TILED, 6)
         for k in weights:
             if k.endswith(("mix.q", "mix.k")):
-                weights[k] = (weights[k].float() * 2.2).bfloat16()
+                weights[k] = (weights[k].float() * 1.4).bfloat16()
         folder, cfg, _ = models("peaked", M.TILED, weights)
         toks = M.tokens(cfg, 290, 5)
         want = models.expect("peaked", toks)
