@@ -6,11 +6,13 @@
 // Pairs are sorted by expert (stable, so results do not depend on timing) and
 // cut into tiles of one expert each; the product kernels take one tile and a
 // block of output channels per workgroup:
-//   expert_tiles   128 pairs x 128 channels through LDS, for many pairs
+//   expert_tiles   128 pairs and 256 channels through LDS, for many pairs
 //   expert_rows    up to 64 pairs, weights straight into registers, for few:
 //                  there the weights' bytes are what counts
 //   expert_plain   any size, bf16 or float
 #include "elem.h"
+
+#include <type_traits>
 
 namespace {
 
@@ -19,31 +21,20 @@ typedef __attribute__((ext_vector_type(16))) float f32x16;
 
 // ---- router ----------------------------------------------------------------
 // The `top` largest of z[0, E) by one wave: experts and sigmoids of their
-// scores, largest first, the lower expert on ties. Overwrites z.
-__device__ void take_top(float* z, int E, int top, int32_t* ids, float* wt) {
-  const int lane = threadIdx.x % WAVE;
-  for (int j = 0; j < top; ++j) {
-    float best = -INFINITY;
-    int at = E;
-    for (int e = lane; e < E; e += WAVE)
-      if (z[e] > best || at == E) {
-        best = z[e];
-        at = e;
-      }
-#pragma unroll
-    for (int o = 32; o > 0; o >>= 1) {
-      const float b = __shfl_xor(best, o, WAVE);
-      const int a = __shfl_xor(at, o, WAVE);
-      if (b > best || (b == best && a < at)) {
-        best = b;
-        at = a;
-      }
+// scores, largest first, the lower expert on ties. An expert's place is the
+// number of experts ahead of it.
+__device__ void take_top(const float* z, int E, int top, int32_t* ids,
+                         float* wt) {
+  for (int e = threadIdx.x % WAVE; e < E; e += WAVE) {
+    const float mine = z[e];
+    int place = 0;
+#pragma unroll 8
+    for (int i = 0; i < E; ++i)
+      place += z[i] > mine || (z[i] == mine && i < e);
+    if (place < top) {
+      ids[place] = e;
+      wt[place] = sigmoid_f(mine);
     }
-    if (lane == 0) {
-      ids[j] = at < E ? at : 0;
-      wt[j] = sigmoid_f(best);
-    }
-    if (at < E && lane == at % WAVE) z[at] = -INFINITY;  // its only reader
   }
 }
 
@@ -81,22 +72,34 @@ __global__ __launch_bounds__(NW * WAVE) void route_kernel(
   float4v acc[ET];
 #pragma unroll
   for (int t = 0; t < ET; ++t) acc[t] = (float4v){0.f, 0.f, 0.f, 0.f};
-  for (int k0 = wave * 64; k0 < K; k0 += NW * 64) {
+  // past the end of K the row counts as zero; experts past E are not looked at
+  const short* wr[ET];
 #pragma unroll
-    for (int s = 0; s < 2; ++s) {
-      const int k = k0 + grp * 16 + s * 8;
-      const short8 a = k < K ? *(const short8*)(h + row * K + k) : zero;
+  for (int t = 0; t < ET; ++t)
+    wr[t] = w + (int64_t)min(t * 16 + col, E - 1) * K;
+  constexpr int AHEAD = ET <= 2 ? 4 : 2;     // steps whose loads go together
+  for (int k0 = wave * 64; k0 < K; k0 += AHEAD * NW * 64) {
+    short8 a[AHEAD][2], b[AHEAD][2][ET];
 #pragma unroll
-      for (int t = 0; t < ET; ++t) {
-        const int e = t * 16 + col;
-        const short8 b = k < K && e < E
-                             ? *(const short8*)(w + (int64_t)e * K + k)
-                             : zero;
-        acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-            __builtin_bit_cast(bf16x8, b), __builtin_bit_cast(bf16x8, a),
-            acc[t], 0, 0, 0);
+    for (int u = 0; u < AHEAD; ++u)
+#pragma unroll
+      for (int s = 0; s < 2; ++s) {
+        const int k = k0 + u * NW * 64 + grp * 16 + s * 8, kc = min(k, K - 8);
+        a[u][s] = *(const short8*)(h + row * K + kc);
+        if (k >= K) a[u][s] = zero;
+#pragma unroll
+        for (int t = 0; t < ET; ++t)
+          b[u][s][t] = *(const short8*)(wr[t] + kc);
       }
-    }
+#pragma unroll
+    for (int u = 0; u < AHEAD; ++u)
+#pragma unroll
+      for (int s = 0; s < 2; ++s)
+#pragma unroll
+        for (int t = 0; t < ET; ++t)
+          acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+              __builtin_bit_cast(bf16x8, b[u][s][t]),
+              __builtin_bit_cast(bf16x8, a[u][s]), acc[t], 0, 0, 0);
   }
 #pragma unroll
   for (int t = 0; t < ET; ++t)
@@ -242,13 +245,11 @@ __global__ __launch_bounds__(256) void expert_rows_kernel(const Pairs p) {
 #pragma unroll
   for (int c = 0; c < 4; ++c)
     wr[c] = (const short*)p.w +
-            ((int64_t)tile.x * N + min(n0 + c * 16 + col, N - 1)) * K +
-            grp * 16;
+            ((int64_t)tile.x * N + min(n0 + c * 16 + col, N - 1)) * K;
 #pragma unroll
   for (int t = 0; t < MT; ++t)
     ar[t] = (const short*)p.a +
-            source<UP>(p, tile.y + min(t * 16 + col, tile.z - 1)) * K +
-            grp * 16;
+            source<UP>(p, tile.y + min(t * 16 + col, tile.z - 1)) * K;
   float4v acc[4][MT];
 #pragma unroll
   for (int c = 0; c < 4; ++c)
@@ -256,18 +257,24 @@ __global__ __launch_bounds__(256) void expert_rows_kernel(const Pairs p) {
     for (int t = 0; t < MT; ++t) acc[c][t] = (float4v){0.f, 0.f, 0.f, 0.f};
   const short8 zero = {0, 0, 0, 0, 0, 0, 0, 0};
   short8 wf[4][2], af[MT][2], wn[4][2], an[MT][2];
+  // past the end of K the pairs' rows count as zero
   auto fetch = [&](int k0) {
 #pragma unroll
     for (int s = 0; s < 2; ++s) {
-      const int k = k0 + s * 8;
-      const bool in = k + grp * 16 < K;
+      const int k = k0 + grp * 16 + s * 8, kc = min(k, K - 8);
 #pragma unroll
-      for (int c = 0; c < 4; ++c)
-        wn[c][s] = in ? *(const short8*)(wr[c] + k) : zero;
+      for (int c = 0; c < 4; ++c) wn[c][s] = *(const short8*)(wr[c] + kc);
 #pragma unroll
-      for (int t = 0; t < MT; ++t)
-        an[t][s] = in && t * 16 + col < tile.z ? *(const short8*)(ar[t] + k)
-                                               : zero;
+      for (int t = 0; t < MT; ++t) {
+        if constexpr (MT > 2) {      // worth leaving absent pairs out
+          an[t][s] = k < K && t * 16 + col < tile.z
+                         ? *(const short8*)(ar[t] + k)
+                         : zero;
+        } else {
+          an[t][s] = *(const short8*)(ar[t] + kc);
+          if (k >= K) an[t][s] = zero;
+        }
+      }
     }
   };
   fetch(wave * 64);
@@ -314,150 +321,194 @@ __global__ __launch_bounds__(256) void expert_rows_kernel(const Pairs p) {
   }
 }
 
-// 128 channels x 128 pairs, K in steps of 64 through two LDS buffers that are
-// filled straight from memory. A row of a step is 128 bytes = 8 pieces; piece
-// c of row r lies at place c ^ (r % 8), so that reads of one piece of 32 rows
-// meet all banks. 4 waves, 64 x 64 each.
-constexpr int BT = 128, BK = 64;
+// 256 channels x 128 pairs, K in steps of 64 through three LDS buffers that are
+// filled straight from memory, two steps ahead. A row of a step is 128 bytes =
+// 8 pieces; piece c of row r lies at place c ^ (r / 2 % 8): the 16 rows a read
+// serves at once then meet all 64 banks. 4 waves, 128 x 64 each, CT x PT tiles
+// of 32 x 32. Loads and LDS reads are spread between the matrix instructions:
+// issued in a row they would hold the wave up.
+constexpr int CT = 4, PT = 2, NB = 3, BK = 64;
+constexpr int TC = 64 * CT, TILE = 64 * PT;
+constexpr int BUF = (TC + TILE) * BK;
+constexpr int TILES_LDS = NB * BUF * (int)sizeof(short);
 constexpr int TG = 8;                // tiles of pairs that run side by side
 
 template <bool UP>
-__global__ __launch_bounds__(256, 2) void expert_tiles_kernel(const Pairs p) {
-  // [buffer][weights, pairs]
-  __shared__ __align__(16) short lds[2][2][BT * BK];
+__global__ __launch_bounds__(256, 1) void expert_tiles_kernel(const Pairs p) {
+  extern __shared__ __align__(16) short tile_lds[];  // NB x [weights, pairs]
   const int N = p.N, K = p.K;
   // Workgroups go round the 8 XCDs in turn: each XCD gets a contiguous share
   // of the work, in which TG tiles of pairs walk the channels together.
-  const int nx = (N + BT - 1) / BT, total = p.tiles[0].x * nx;
+  const int nx = (N + TC - 1) / TC, total = p.tiles[0].x * nx;
   const int share = (total + 7) / 8;
   const int id = blockIdx.x % 8 * share + blockIdx.x / 8;
   if ((int)blockIdx.x / 8 >= share || id >= total) return;
   const int g = id / (TG * nx), in = id % (TG * nx);
   const int width = min(TG, p.tiles[0].x - g * TG);
   const int4 tile = p.tiles[1 + g * TG + in % width];
-  const int n0 = in / width * BT;
+  const int n0 = in / width * TC;
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
   const int col = lane & 31, hi = lane >> 5;
   const int wc = wave & 1, wp = wave >> 1;    // its channels, its pairs
 
-  // a wave fills rows 32 wave .. + 31 of both: 8 rows per instruction
-  const short *wsrc[4], *asrc[4];
-  const int piece = (lane % 8) ^ (lane / 8);
+  // A wave fills a quarter of the rows of both, 8 rows per instruction, from
+  // byte offsets within the expert's weights and p.a (both under 4 GiB).
+  // Rows past the tile repeat its last one: they are computed and dropped.
+  constexpr int LW = 2 * CT, LOADS = 2 * CT + 2 * PT;
+  const char* wbase = (const char*)p.w + (int64_t)tile.x * N * K * 2;
+  const char* abase = (const char*)p.a;
+  uint32_t src[LOADS];
+  int64_t rows[2 * PT];
 #pragma unroll
-  for (int j = 0; j < 4; ++j) {
-    const int r = wave * 32 + j * 8 + lane / 8;
-    wsrc[j] = (const short*)p.w +
-              ((int64_t)tile.x * N + min(n0 + r, N - 1)) * K + piece * 8;
-    asrc[j] = (const short*)p.a +
-              source<UP>(p, tile.y + min(r, tile.z - 1)) * K + piece * 8;
-  }
-  auto stage = [&](int buf, int k0) {
+  for (int j = 0; j < 2 * PT; ++j)
+    rows[j] = source<UP>(p, tile.y + min(wave * 16 * PT + j * 8 + lane / 8,
+                                         tile.z - 1));
+  auto piece = [&](int j) {
+    return (lane % 8 ^ (lane / 16 + j % 2 * 4)) * 8;
+  };
+#pragma unroll
+  for (int j = 0; j < LW; ++j)
+    src[j] = ((uint32_t)min(n0 + wave * 16 * CT + j * 8 + lane / 8, N - 1) *
+                  K + piece(j)) * 2;
+  const int steps = K / BK;
+  auto column = [&](int s) { return min(s, steps - 1) * BK * 2; };
+  auto load = [&](int buf, int k, int j) {
     typedef __attribute__((address_space(1))) const unsigned int gmem;
     typedef __attribute__((address_space(3))) unsigned int smem;
-#pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      __builtin_amdgcn_global_load_lds(
-          (gmem*)(wsrc[j] + k0),
-          (smem*)(&lds[buf][0][(wave * 32 + j * 8) * BK]), 16, 0, 0);
-      __builtin_amdgcn_global_load_lds(
-          (gmem*)(asrc[j] + k0),
-          (smem*)(&lds[buf][1][(wave * 32 + j * 8) * BK]), 16, 0, 0);
-    }
+    const int row = j < LW ? wave * 16 * CT + j * 8
+                           : TC + wave * 16 * PT + (j - LW) * 8;
+    __builtin_amdgcn_global_load_lds(
+        (gmem*)((j < LW ? wbase : abase) + k + src[j]),
+        (smem*)(tile_lds + buf * BUF + row * BK), 16, 0, 0);
   };
-  f32x16 acc[2][2];
 #pragma unroll
-  for (int c = 0; c < 2; ++c)
+  for (int j = 0; j < LW; ++j) load(0, column(0), j);
 #pragma unroll
-    for (int t = 0; t < 2; ++t) acc[c][t] = (f32x16)(0.f);
-  asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-  stage(0, 0);
-  const int steps = K / BK;
+  for (int j = 0; j < 2 * PT; ++j)
+    src[LW + j] = ((uint32_t)rows[j] * K + piece(j)) * 2;
+#pragma unroll
+  for (int j = LW; j < LOADS; ++j) load(0, column(0), j);
+#pragma unroll
+  for (int j = 0; j < LOADS; ++j) load(1, column(1), j);
+
+  f32x16 acc[CT][PT];
+#pragma unroll
+  for (int c = 0; c < CT; ++c)
+#pragma unroll
+    for (int t = 0; t < PT; ++t) acc[c][t] = (f32x16)(0.f);
+  int buf = 0, fill = NB - 1;
   for (int s = 0; s < steps; ++s) {
-    const int buf = s & 1;
-    // this step has landed, and the other buffer is no longer read
-    asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)" ::: "memory");
+    // this step has landed (the next may be on its way), and the buffer that
+    // is filled now is no longer read
+    asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)" ::"i"(LOADS) : "memory");
     __builtin_amdgcn_s_barrier();
     asm volatile("" ::: "memory");
-    if (s + 1 < steps) stage(buf ^ 1, (s + 1) * BK);
-    const short *wl = &lds[buf][0][(wc * 64 + col) * BK],
-                *al = &lds[buf][1][(wp * 64 + col) * BK];
+    const int k = column(s + NB - 1);          // the last step repeats
+    const short* wl = tile_lds + buf * BUF + (wc * 32 * CT + col) * BK;
+    const short* al = tile_lds + buf * BUF + (TC + wp * 32 * PT + col) * BK;
+    bf16x8 wf[2][CT], af[2][PT];
+    auto read = [&](int x, int kk) {
+      const int at = ((kk * 2 + hi) ^ (col / 2 & 7)) * 8;
+#pragma unroll
+      for (int c = 0; c < CT; ++c)
+        wf[x][c] = *(const bf16x8*)(wl + c * 32 * BK + at);
+#pragma unroll
+      for (int t = 0; t < PT; ++t)
+        af[x][t] = *(const bf16x8*)(al + t * 32 * BK + at);
+    };
+    read(0, 0);
+    __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
     for (int kk = 0; kk < BK / 16; ++kk) {
-      const int at = ((kk * 2 + hi) ^ (col & 7)) * 8;
-      bf16x8 wf[2], af[2];
+      const bool more = kk + 1 < BK / 16;
+      if (more) read(kk + 1 & 1, kk + 1);
 #pragma unroll
-      for (int c = 0; c < 2; ++c) {
-        wf[c] = *(const bf16x8*)(wl + c * 32 * BK + at);
-        af[c] = *(const bf16x8*)(al + c * 32 * BK + at);
-      }
+      for (int j = 0; j < LOADS / 4; ++j) load(fill, k, kk * LOADS / 4 + j);
 #pragma unroll
-      for (int c = 0; c < 2; ++c)
+      for (int c = 0; c < CT; ++c)
 #pragma unroll
-        for (int t = 0; t < 2; ++t)
+        for (int t = 0; t < PT; ++t)
           acc[c][t] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(
-              wf[c], af[t], acc[c][t], 0, 0, 0);
-    }
-  }
+              wf[kk & 1][c], af[kk & 1][t], acc[c][t], 0, 0, 0);
+      // the order: matrix, read, (load), ... matrix
 #pragma unroll
-  for (int t = 0; t < 2; ++t) {
-    const int i = wp * 64 + t * 32 + col;
-    if (i >= tile.z) continue;
-    const int pair = p.order[tile.y + i];
-    const float wt = UP ? p.weights[pair] : 1.f;
-    short* o = (short*)p.out + (int64_t)(UP ? tile.y + i : pair) * N;
-#pragma unroll
-    for (int c = 0; c < 2; ++c)
-#pragma unroll
-      for (int q = 0; q < 4; ++q) {
-        const int n = n0 + wc * 64 + c * 32 + q * 8 + hi * 4;
-        if (n >= N) continue;
-        const f32x16& v = acc[c][t];
-        *(short4v*)(o + n) =
-            (short4v){f32_to_bf16(finish<UP>(p, v[4 * q], wt)),
-                      f32_to_bf16(finish<UP>(p, v[4 * q + 1], wt)),
-                      f32_to_bf16(finish<UP>(p, v[4 * q + 2], wt)),
-                      f32_to_bf16(finish<UP>(p, v[4 * q + 3], wt))};
+      for (int i = 0; i < CT + PT; ++i) {
+        __builtin_amdgcn_sched_group_barrier(0x008, 1, 0);
+        if (more) __builtin_amdgcn_sched_group_barrier(0x100, 1, 0);
+        if (i % 2 == 0) __builtin_amdgcn_sched_group_barrier(0x020, 1, 0);
       }
+      __builtin_amdgcn_sched_group_barrier(0x008, CT * PT - CT - PT, 0);
+      __builtin_amdgcn_sched_barrier(0);
+    }
+    buf = buf + 1 == NB ? 0 : buf + 1;
+    fill = fill + 1 == NB ? 0 : fill + 1;
   }
+  asm volatile("s_waitcnt vmcnt(0)" ::: "memory");   // the repeated loads
+
+  auto write = [&](auto act) {
+#pragma unroll
+    for (int t = 0; t < PT; ++t) {
+      const int i = wp * 32 * PT + t * 32 + col;
+      if (i >= tile.z) continue;
+      const int pair = p.order[tile.y + i];
+      const float wt = UP ? p.weights[pair] : 1.f;
+      short* o = (short*)p.out + (int64_t)(UP ? tile.y + i : pair) * N;
+#pragma unroll
+      for (int c = 0; c < CT; ++c)
+#pragma unroll
+        for (int q = 0; q < 4; ++q) {
+          const int n = n0 + wc * 32 * CT + c * 32 + q * 8 + hi * 4;
+          if (n >= N) continue;
+          short4v v;
+#pragma unroll
+          for (int x = 0; x < 4; ++x) {
+            const float f = acc[c][t][4 * q + x];
+            v[x] = f32_to_bf16(UP ? activate(act, f * wt) : f);
+          }
+          *(short4v*)(o + n) = v;
+        }
+    }
+  };
+  using std::integral_constant;
+  if (!UP || p.act == ACT_RELU_SQUARED)
+    write(integral_constant<int, ACT_RELU_SQUARED>{});
+  else if (p.act == ACT_SILU)
+    write(integral_constant<int, ACT_SILU>{});
+  else
+    write(integral_constant<int, ACT_GELU_TANH>{});
 }
 
-enum Form { PLAIN, ROWS, TILES };
-
-Form form(int f32, int plain, int tile, int N, int K) {
-  if (f32 || plain || N % 8 || K % 8) return PLAIN;
-  return tile == BT && K % BK == 0 ? TILES : ROWS;
+template <bool UP>
+hipError_t launch_tiles(const Pairs& p, int max_tiles, hipStream_t stream) {
+  // every XCD's share is rounded up
+  const int64_t n = ((int64_t)max_tiles * ((p.N + TC - 1) / TC) + 7) / 8 * 8;
+  if (n > 0x7fffffff || p.N % 8 || p.K % BK || p.K < 2 * BK ||
+      (int64_t)p.N * p.K >= 1ll << 31)
+    return hipErrorInvalidValue;
+  auto fn = expert_tiles_kernel<UP>;
+  hipError_t e = hipFuncSetAttribute(
+      (const void*)fn, hipFuncAttributeMaxDynamicSharedMemorySize, TILES_LDS);
+  if (e != hipSuccess) return e;
+  hipLaunchKernelGGL(fn, dim3((uint32_t)n), dim3(256), TILES_LDS, stream, p);
+  HIP_CHECK_LAST();
+  return hipSuccess;
 }
 
 template <bool UP>
 hipError_t product(int f32, int plain, int tile, int max_tiles, const Pairs& p,
                    hipStream_t stream) {
-  const Form f = form(f32, plain, tile, p.N, p.K);
-  const dim3 block(256);
-  if (f == TILES) {
-    // every XCD's share is rounded up
-    const int64_t n = ((int64_t)max_tiles * ((p.N + BT - 1) / BT) + 7) / 8 * 8;
-    if (n > 0x7fffffff) return hipErrorInvalidValue;
-    hipLaunchKernelGGL(expert_tiles_kernel<UP>, dim3((uint32_t)n), block, 0,
-                       stream, p);
-  } else {
-    const dim3 grid((p.N + 63) / 64, max_tiles);
-    if (max_tiles > 65535) return hipErrorInvalidValue;
-    if (f == PLAIN && f32)
-      hipLaunchKernelGGL((expert_plain_kernel<float, UP>), grid, block, 0,
-                         stream, p);
-    else if (f == PLAIN)
-      hipLaunchKernelGGL((expert_plain_kernel<short, UP>), grid, block, 0,
-                         stream, p);
-    else if (tile <= 16)
-      hipLaunchKernelGGL((expert_rows_kernel<1, UP>), grid, block, 0, stream,
-                         p);
-    else if (tile <= 32)
-      hipLaunchKernelGGL((expert_rows_kernel<2, UP>), grid, block, 0, stream,
-                         p);
-    else
-      hipLaunchKernelGGL((expert_rows_kernel<4, UP>), grid, block, 0, stream,
-                         p);
-  }
+  if (tile == TILE) return launch_tiles<UP>(p, max_tiles, stream);
+  const dim3 grid((p.N + 63) / 64, max_tiles), block(256);
+  if (max_tiles > 65535 || tile > 64) return hipErrorInvalidValue;
+#define GO(KERNEL) hipLaunchKernelGGL((KERNEL), grid, block, 0, stream, p)
+#define K2(NAME, ARG) NAME<ARG, UP>
+  if (f32) GO(K2(expert_plain_kernel, float));
+  else if (plain || p.N % 8 || p.K % 8) GO(K2(expert_plain_kernel, short));
+  else if (tile <= 16) GO(K2(expert_rows_kernel, 1));
+  else if (tile <= 32) GO(K2(expert_rows_kernel, 2));
+  else GO(K2(expert_rows_kernel, 4));
+#undef K2
+#undef GO
   HIP_CHECK_LAST();
   return hipSuccess;
 }
@@ -489,20 +540,25 @@ hipError_t lds_route(int f32, const void* h, const void* w, int32_t* ids,
                      dim3((uint32_t)((rows + 15) / 16)), dim3(NW * WAVE),     \
                      NW * 256 * ET * sizeof(float), stream, (const short*)h,  \
                      (const short*)w, ids, wt, rows, K, E, top)
-  if (E <= 16) GO(1, 8); else if (E <= 32) GO(2, 8);
-  else if (E <= 64) GO(4, 8); else if (E <= 128) GO(8, 8);
+  if (E <= 16) GO(1, 16); else if (E <= 32) GO(2, 16);
+  else if (E <= 64) GO(4, 16); else if (E <= 128) GO(8, 8);
   else GO(16, 4);
 #undef GO
   HIP_CHECK_LAST();
   return hipSuccess;
 }
 
-// pairs of one expert that a workgroup takes
-int lds_expert_tile(int f32, int plain, int P, int E, int N, int K) {
+// pairs of one expert that a workgroup takes: about as many as an expert has
+int lds_expert_tile(int f32, int plain, int P, int T, int E, int N, int K) {
   const int per = (P + E - 1) / E;
-  if (f32 || plain) return 16;
-  return per <= 12 ? 16 : per <= 24 ? 32
-         : per <= 48 || N % BK || K % BK ? 64 : BT;
+  const int64_t limit = 1ll << 31;      // elements: offsets stay under 4 GiB
+  if (f32 || plain || per <= 12) return 16;
+  if (per <= 24) return 32;
+  if (per <= 48 || N % BK || K % BK || N < 2 * BK || K < 2 * BK ||
+      (int64_t)N * K >= limit || (int64_t)T * K >= limit ||
+      (int64_t)P * N >= limit)
+    return 64;
+  return TILE;
 }
 
 // tiles of P pairs at most

@@ -18,7 +18,7 @@ hipError_t lds_grouped_prefill(const void*, int64_t, const void*,
                                float, int, float, hipStream_t);
 hipError_t lds_route(int, const void*, const void*, int32_t*, float*, int64_t,
                      int, int, int, hipStream_t);
-int lds_expert_tile(int, int, int, int, int, int);
+int lds_expert_tile(int, int, int, int, int, int, int);
 int lds_expert_max_tiles(int, int, int);
 hipError_t lds_sort_pairs(const int32_t*, int32_t*, void*, int, int, int,
                           hipStream_t);
@@ -195,7 +195,8 @@ Tensor experts(Tensor h, Tensor ids, Tensor weights, Tensor up, Tensor down,
               "experts");
   auto out = torch::empty({P, K}, h.options());
   if (P == 0) return out;
-  const int tile = lds_expert_tile(f32, plain, (int)P, (int)E, (int)F, (int)K);
+  const int tile = lds_expert_tile(f32, plain, (int)P, (int)T, (int)E, (int)F,
+                                   (int)K);
   const int max_tiles = lds_expert_max_tiles((int)P, (int)E, tile);
   auto order = torch::empty({P}, ids.options());
   auto tiles = torch::empty({1 + max_tiles, 4}, ids.options());
