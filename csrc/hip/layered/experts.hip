@@ -120,6 +120,19 @@ __global__ __launch_bounds__(NW * WAVE) void route_kernel(
 // ---- sorting ---------------------------------------------------------------
 constexpr int ST = 1024, SV = 8;   // threads; pairs per thread and sweep
 
+// SV experts from place i on; -1 past the end (i is a multiple of SV)
+__device__ __forceinline__ void load_ids(const int32_t* ids, int i, int P,
+                                         int* x) {
+  if (i + SV <= P) {
+    const int4 a = *(const int4*)(ids + i), b = *(const int4*)(ids + i + 4);
+    x[0] = a.x; x[1] = a.y; x[2] = a.z; x[3] = a.w;
+    x[4] = b.x; x[5] = b.y; x[6] = b.z; x[7] = b.w;
+  } else {
+#pragma unroll
+    for (int j = 0; j < SV; ++j) x[j] = i + j < P ? ids[i + j] : -1;
+  }
+}
+
 // One workgroup per expert. order [P]: pairs by expert; tiles [1 + max_tiles]
 // = (number of tiles, ..), then (expert, first place in order, pairs, 0).
 __global__ __launch_bounds__(ST) void sort_pairs_kernel(
@@ -131,9 +144,12 @@ __global__ __launch_bounds__(ST) void sort_pairs_kernel(
   const int wave = tid / WAVE, lane = tid % WAVE;
   for (int i = tid; i < E; i += ST) hist[i] = 0;
   __syncthreads();
-  for (int i = tid; i < P; i += ST) {
-    const int x = ids[i];
-    if (x >= 0 && x < E) atomicAdd(&hist[x], 1);
+  for (int i = tid * SV; i < P; i += ST * SV) {
+    int x[SV];
+    load_ids(ids, i, P, x);
+#pragma unroll
+    for (int j = 0; j < SV; ++j)
+      if (x[j] >= 0 && x[j] < E) atomicAdd(&hist[x[j]], 1);
   }
   __syncthreads();
   if (wave == 0) {                     // pairs and tiles of lower experts
@@ -161,10 +177,10 @@ __global__ __launch_bounds__(ST) void sort_pairs_kernel(
   int base = first;
   for (int i0 = 0; i0 < P; i0 += ST * SV) {   // workgroup-uniform
     const int i = i0 + tid * SV;
-    int mine = 0;
+    int mine = 0, x[SV];
+    load_ids(ids, i, P, x);
 #pragma unroll
-    for (int j = 0; j < SV; ++j)
-      if (i + j < P && ids[i + j] == e) mine |= 1 << j;
+    for (int j = 0; j < SV; ++j) mine |= (x[j] == e) << j;
     const int n = __popc(mine);
     int before = n;                    // inclusive sum over the wave
 #pragma unroll
